@@ -263,22 +263,17 @@ class Runner:
             out = torch.einsum("eth,te->th", y.float(), wfull)
             return out.to(x.dtype)
 
-        import os as _os
-
         use_grouped = (
             x.device.type == "cuda"
             and x.dtype == torch.bfloat16  # the kernel's only instantiation
             and H % 128 == 0 and I % 128 == 0
             and T <= self.MOE_GROUPED_ROWS * E // top_k
-            and _os.environ.get("BEE2BEE_MOE_BMM") != "1"
         )
-        # the padded bmm stays CPU-only (and opt-in for A/B measurement):
-        # hipBLASLt's batched TN bf16 kernel memory-faults on gfx950 once
-        # the padded M reaches ~1K (repro: scripts/debug_moe_t4096.py, C
-        # 1049 AND 1056) — GPU sizes above the grouped range take the
-        # per-expert GEMM loop below, whose plain TN GEMMs are solid
-        use_bmm = (x.device.type != "cuda"
-                   or _os.environ.get("BEE2BEE_MOE_BMM") == "1")
+        # the padded bmm is CPU-only: the library's batched TN bf16 product
+        # is not usable on gfx950 at these sizes — GPU sizes above the
+        # grouped range take the per-expert GEMM loop below, whose plain TN
+        # GEMMs are solid
+        use_bmm = x.device.type != "cuda"
         if T <= self.MOE_BMM_MAX_TOKENS and (use_grouped or use_bmm):
             # counting sort from one-hot cumsums: every op here (one_hot,
             # cumsum, gather, index_copy) is hipGraph-capture-safe —
@@ -308,9 +303,7 @@ class Runner:
                 # padded per-expert bmm: weights read once per expert, flops
                 # proportional to max routed count; counts.max() is one host
                 # sync per MoE layer (so no hipGraph above the dense range).
-                # M aligns up to 16: odd M (e.g. 1049) faults hipBLASLt's
-                # TN bf16 batched kernel on gfx950 (repro:
-                # scripts/debug_moe_t4096.py; <2% padded flops)
+                # M aligns up to 16 (<2% padded flops)
                 C = (int(counts.max()) + 15) & ~15
                 padded = torch.zeros(E, C, H, dtype=x.dtype, device=x.device)
                 padded[flat_e, rank] = x[tok]
