@@ -25,6 +25,8 @@ the SAME page and slot bookkeeping:
     whole-width conv, the q|k|v projection for a delta mixer's short conv);
   * grouped-query attention with a short convolution on its projected
     q|k|v: the two page pools and the last taps-1 projected rows per slot;
+  * grouped-query attention whose values are normed per head: normed when
+    cached;
   * an element-wise gated recurrence (minGRU): state [n_slots, width] fp32;
   * a parallel mixer (attention + delta rule or minGRU side by side) has
     pages AND state in the same layer.

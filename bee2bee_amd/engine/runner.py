@@ -90,6 +90,12 @@ class Runner:
         return ops.fused_add_rmsnorm(x, resid, w, self.spec.rms_eps)
 
     def lm_head(self, hidden: torch.Tensor) -> torch.Tensor:
+        if self.spec.is_hybrid and self.spec.norm_type == "tanh":
+            # fp32 residual stream; the logit scale is in the norm's numbers
+            normed = ops.add_tanh_norm(
+                hidden.contiguous(), None, None,
+                self.weights.final_tanh_scaled, self.dtype)
+            return F.linear(normed, self.weights.lm_head)
         if self.spec.is_hybrid and self.spec.norm_type == "group_rmsnorm":
             # fp32 residual stream, weighted grouped final norm
             normed = ops.add_group_rmsnorm(
@@ -248,11 +254,22 @@ class Runner:
             weights, idx = ops.group_topk_gate(
                 logits, top_k, ffn.n_groups, ffn.keep_groups,
                 "sigmoid" if ffn.score == "sigmoid_all" else "softmax",
-                ffn.group_top)
+                ffn.group_top,
+                lw.moe_choice_bias if ffn.choice_bias else None, ffn.renorm,
+                ffn.route_scale)
         else:
             weights, idx = ops.moe_topk_gate(logits, top_k)  # [T,k]
         T, H = x.shape
 
+        if (lw.moe_w_down_cat is not None and ffn.act == "silu_glu"
+                and T <= self.MOE_DENSE_MAX_TOKENS):
+            # every expert's columns as two plain products: gate|up of all
+            # experts, then activation * routing weight (zero for experts a
+            # token did not choose) against the experts' output matrices
+            # side by side, which sums the experts in the fp32 accumulator
+            gu = F.linear(x, lw.moe_w_gate_up.view(E * U, H))
+            act = ops.routed_silu_glu(gu.view(T, E, U), weights, idx)
+            return F.linear(act, lw.moe_w_down_cat)
         if T <= self.MOE_DENSE_MAX_TOKENS:
             x_e = x.unsqueeze(0).expand(E, T, H)
             gu = torch.bmm(x_e, lw.moe_w_gate_up.transpose(1, 2))  # [E,T,2I]
@@ -484,6 +501,8 @@ class Runner:
             return self._forward_sandwich_w(x, meta)
         if s.layer_specs[0].form == "parallel_gated":
             return self._forward_parallel_gated(x, meta)
+        if s.layer_specs[0].form == "sandwich_tanh":
+            return self._forward_sandwich_tanh(x, meta)
         if s.layer_specs[0].form == "parallel":
             # x += mixer(h) + ffn(h), h = unit(x) * w: the residual add and
             # the next layer's norm run as one kernel
@@ -643,6 +662,49 @@ class Runner:
                       cu, lw.talk, gate, m.window, out, max_qlen)
         return F.linear(out, lw.wo)
 
+    # -------------------------------------------------- dynamic-tanh layers
+
+    def _forward_sandwich_tanh(self, x: torch.Tensor, meta) -> torch.Tensor:
+        """x += n1b(mixer(n1(x))); x += n2b(ffn(n2(x))) with n(x) =
+        tanh(alpha x) * w + b. Post-norm, residual add and the next pre-norm
+        are ONE element-wise kernel."""
+        s, W, dt = self.spec, self.weights, self.dtype
+        n = s.n_layers
+        normed = ops.add_tanh_norm(x, None, None, W.layers[0].norms[0], dt)
+        for i in range(n):
+            lw, l = W.layers[i], s.layer_specs[i]
+            nxt = W.layers[i + 1].norms[0] if i + 1 < n else None
+            y = self._mixer_part(i, l.mixer, lw, normed, meta)
+            if l.ffn is not None:
+                normed = ops.add_tanh_norm(x, y, lw.norms[1], lw.norms[2], dt)
+                y = self._moe_mlp(lw, normed, ffn=l.ffn)
+            normed = ops.add_tanh_norm(x, y, lw.norms[-1], nxt, dt)
+            if self.layer_tap is not None:
+                self.layer_tap(i, x)
+        return x
+
+    def _mixer_part(self, i: int, m, lw, h: torch.Tensor, meta
+                    ) -> torch.Tensor:
+        """A single mixer of layer i on the normed input h: one fused input
+        projection, the mixer's kernels, its output projection."""
+        ins, _ = lw.layout
+        proj = F.linear(h, lw.w_in, lw.b_in)
+
+        def cols(key):
+            off, n = ins[key]
+            return proj[:, off : off + n]
+
+        ns = lw.mix[""]
+        if m.kind == "gqa_attention":
+            o = self._gqa_attn_part(i, m, ns, cols, "", meta)
+        elif m.kind == "latent_attention":
+            o = self._latent_attn_part(i, m, ns, cols, "", meta)
+        else:
+            o = torch.empty(h.shape[0], m.out_size, dtype=self.dtype,
+                            device=h.device)
+            self._delta_part(i, m, ns, cols, "", meta, o, 1.0)
+        return F.linear(o, ns.wo)
+
     # ------------------------------------------ gated parallel-form layers
 
     def _forward_parallel_gated(self, x: torch.Tensor, meta) -> torch.Tensor:
@@ -715,8 +777,9 @@ class Runner:
 
     def _gqa_attn_part(self, i: int, m, ns, cols, pre, meta) -> torch.Tensor:
         """Grouped-query attention of layer run i: optional short conv on
-        the projected q|k|v (fp32 out), rotation + page store, attention
-        with the spec's cap / score mix / sink / window / head gate."""
+        the projected q|k|v (fp32 out), rotation (or the norm over the whole
+        projection) + page store, attention with the spec's cap / score mix
+        / sink / window / distance bias / head gate."""
         (positions, slot_mapping, cu, seq_idx, block_table, state_slots,
          max_qlen) = meta
         T = positions.shape[0]
@@ -737,15 +800,23 @@ class Runner:
             cos, sin = self._rope_tables(m.rope_dims, m.rope_base, f64=True,
                                          scaling=m.rope_scaling)
         k_cache, v_cache = self.kv.k_cache[i], self.kv.v_cache[i]
-        # the query leaves this rotated and times the score scale
+        # the query leaves this rotated (or normed) and times the score scale
         if q.dtype == self.dtype:
             q_out = q
         else:
             q_out = torch.empty(T, m.heads, m.dim, dtype=self.dtype,
                                 device=q.device)
-        ops.rope_store(q, k, v, q_out, m.rope_dims,
-                       m.rope_layout == "interleaved", positions, cos, sin,
-                       m.scale, k_cache, v_cache, slot_mapping)
+        if m.proj_norm:
+            if m.rope_dims or ns.conv_w is not None:
+                raise ValueError("a norm over the whole projection does not "
+                                 "combine with a rotation or a convolution")
+            ops.proj_norm_store(q, k, v, ns.q_norm, ns.k_norm, m.v_norm,
+                                self.spec.rms_eps, m.scale, k_cache, v_cache,
+                                slot_mapping)
+        else:
+            ops.rope_store(q, k, v, q_out, m.rope_dims,
+                           m.rope_layout == "interleaved", positions, cos,
+                           sin, m.scale, k_cache, v_cache, slot_mapping)
         sink = None
         if m.zero_sink:
             sink = self._zeros_f32(m.heads)
@@ -753,7 +824,7 @@ class Runner:
         ops.gqa_attn(q_out, k_cache, v_cache, block_table, positions, seq_idx,
                      cu, m.softcap, ns.talk if m.score_mix else None, sink,
                      cols(pre + "g") if m.head_gate else None, m.window, out,
-                     max_qlen)
+                     max_qlen, dist=ns.dist)
         return out
 
     def _zeros_f32(self, n: int) -> torch.Tensor:
@@ -768,7 +839,8 @@ class Runner:
         """Latent attention of layer run i in absorbed form (the key
         up-projection folded into the query, the value up-projection into
         the output), queries through their own normed latent when the spec
-        has one, a per-head sink and sigmoid head gate in the kernel."""
+        has one, an optional per-head sink and sigmoid head gate in the
+        kernel."""
         (positions, slot_mapping, cu, seq_idx, block_table, _,
          max_qlen) = meta
         T, H = positions.shape[0], m.heads
@@ -779,12 +851,14 @@ class Runner:
             q = F.linear(cq, ns.w_uq).view(T, H, D + R)
         else:
             q = cols(pre + "q").view(T, H, D + R)
-        kv, gate = cols(pre + "dkv"), cols(pre + "g")
+        kv = cols(pre + "dkv")
+        gate = cols(pre + "g") if m.head_gate else None
         cache = self.kv.k_cache[i]
-        cos, sin = self._rope_tables(m.rope_dims, m.rope_base, f64=True)
+        cos, sin = self._rope_tables(m.rope_dims, m.rope_base, f64=True,
+                                     scaling=m.rope_scaling)
         ops.latent_rope_store(q[..., D:], kv, ns.kv_norm, self.spec.rms_eps,
                               C, m.rope_dims, positions, cos, sin, cache,
-                              slot_mapping)
+                              slot_mapping, m.rope_layout == "interleaved")
         q_abs = torch.bmm(q[..., :D].transpose(0, 1), ns.w_uk)    # [H,T,C]
         lat = ops.latent_attn(q_abs, q[..., D:], gate, cache, block_table,
                               positions, seq_idx, cu, m.window, m.scale,

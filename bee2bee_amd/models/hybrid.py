@@ -47,6 +47,16 @@ added back before every later pass):
   rot.{base, dims, scaling.{factor}}}, mixer.right.{width},
   layers[i].mlp.{kind: moe, expert.ff, router.{experts, top,
   groups.{count, keep}}} (or null).
+
+Tudatar config.json keys (dynamic-tanh norms before and after each sublayer):
+  architecture, vocab, width, norm.eps, logit_scale,
+  layers[i].type in {latent_attention, attention, channel_delta},
+  latent_attention: mixer.{heads, dim, rot_dim, vdim, kv_rank, q_rank, scale,
+  rot.{base, dims, scaling.{factor, original, fast, slow}}},
+  attention: mixer.{heads, kv_heads, dim, vdim, scale, mask.size},
+  channel_delta: mixer.{heads, kv_heads, dim, vdim, conv},
+  layers[i].mlp.{kind: moe, expert.ff, router.{experts, top, scale}} (or
+  null).
 """
 from __future__ import annotations
 
@@ -74,14 +84,21 @@ class LatentAttnSpec:
     # a learned logit per head that counts once in the softmax denominator
     # and has neither key nor value
     sink: bool = False
+    # a sigmoid gate per head on the output
+    head_gate: bool = True
+    # rotated pairs: "half" (i, i + rope_dims/2) or "interleaved" (2i, 2i+1);
+    # rope_scaling: None or {factor, original, fast, slow}
+    rope_layout: str = "half"
+    rope_scaling: Optional[Dict[str, float]] = None
 
     kind = "latent_attention"
 
     @property
     def in_sizes(self) -> Tuple[Tuple[str, int], ...]:
         """Rows of the fused input projection, in order."""
-        return (("dq" if self.q_rank else "q", self.q_rank or self.q_size),
-                ("dkv", self.cache_dim), ("g", self.heads))
+        out = (("dq" if self.q_rank else "q", self.q_rank or self.q_size),
+               ("dkv", self.cache_dim))
+        return out + ((("g", self.heads),) if self.head_gate else ())
 
     @property
     def out_size(self) -> int:
@@ -252,6 +269,12 @@ class GqaAttnSpec:
     BEFORE the softmax (score_mix), a sliding window (0: none), a
     zero-logit sink in the softmax denominator (zero_sink: one is added to
     the sum), and a sigmoid gate per head on the output (head_gate).
+    proj_norm: queries and keys RMS-normed over ALL rows of their projection
+    at once (before the split into heads), with a weight per row; v_norm:
+    each head's value divided by its root mean square before it is cached.
+    distance_bias: a_h ln(1 + b_h (i - j)) is taken off every scaled score,
+    a_h and b_h learned per head. bias covers q, k, v and, unless out_bias
+    is off, the output projection.
     rope_scaling: None, {"kind": "linear", "factor"} (every frequency
     divided by factor) or {"kind": "banded", "factor", "low", "high",
     "original"} (wavelengths above original/low slowed by factor, below
@@ -272,6 +295,10 @@ class GqaAttnSpec:
     bias: bool = False
     taps: int = 0
     head_gate: bool = False
+    proj_norm: bool = False
+    v_norm: bool = False
+    distance_bias: bool = False
+    out_bias: bool = True
 
     kind = "gqa_attention"
 
@@ -360,7 +387,10 @@ class MoEFFNSpec:
     with scores = sigmoid of each logit. group_top: a group's score is the
     sum of its group_top largest expert scores.
     act "gelu": experts without a gate, y = down(gelu(up h)), exact (erf)
-    gelu."""
+    gelu.
+    choice_bias: a learned number per expert joins the scores for the choice
+    only. renorm: the chosen scores are divided by their sum (+ 1e-20);
+    route_scale multiplies the weights last."""
     n_experts: int
     top_k: int
     ff: int
@@ -373,6 +403,9 @@ class MoEFFNSpec:
     n_groups: int = 1
     keep_groups: int = 1
     group_top: int = 1
+    choice_bias: bool = False
+    renorm: bool = False
+    route_scale: float = 1.0
 
     @property
     def up_rows(self) -> int:
@@ -387,6 +420,8 @@ class LayerSpec:
     # "sandwich": scalar-gain norms before and after each sublayer, mixer
     # then feed-forward. "parallel": x += mixer(h) + ffn(h), h = norm(x) * w.
     # "sandwich_w": as "sandwich" with weighted, grouped RMS norms.
+    # "sandwich_tanh": as "sandwich" with dynamic-tanh norms,
+    # tanh(alpha x) * w + b (no row statistics).
     # "parallel_gated": x += sigmoid(W1 h + b1) * mixer(h)
     #                      + sigmoid(W2 h + b2) * ffn(h), h = norm(x) * w.
     form: str = "sandwich"
@@ -693,13 +728,67 @@ def gated_layer_specs_from_cfg(layers: List[Dict[str, Any]],
     return out
 
 
-def gated_layout(l: LayerSpec, width: int
-                 ) -> Tuple[Dict[str, Tuple[int, int]], int]:
-    """Rows of a gated parallel-form layer's ONE input matrix: every
-    projection that reads the normed h — the mixer's (per part, in in_sizes
-    order), then the two residual gates 'rg1' (mixer) and 'rg2'
-    (feed-forward, when there is one). Every segment starts on a multiple of
-    8 rows. Returns ({name: (offset, size)}, total)."""
+def _tudatar_mixer_from_cfg(kind: str, m: Dict[str, Any]):
+    if kind == "attention":
+        spec = _gqa_attn_from_cfg(m, bias=True, out_bias=False,
+                                  proj_norm=True, v_norm=True,
+                                  distance_bias=True)
+        spec.rope_dims = 0          # positions enter through the bias only
+        return spec
+    if kind == "channel_delta":
+        return _delta_from_cfg(m, channel_decay=True, gate="sigmoid")
+    if kind == "latent_attention":
+        rot = m.get("rot") or {}
+        rot_dim = int(m["rot_dim"])
+        dims = int(rot.get("dims", rot_dim))
+        if dims % 2 or dims > rot_dim:
+            raise ValueError("latent attention: rot.dims must be even and "
+                             "<= rot_dim")
+        sc = rot.get("scaling") or None
+        if sc is not None:
+            sc = {k: float(sc[k])
+                  for k in ("factor", "original", "fast", "slow")}
+        return LatentAttnSpec(
+            heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=rot_dim,
+            vdim=int(m["vdim"]), kv_rank=int(m["kv_rank"]),
+            window=int((m.get("mask") or {}).get("size", 0) or 0),
+            rope_base=float(rot.get("base", 10000.0)), rope_dims=dims,
+            scale=float(m["scale"]), q_rank=int(m.get("q_rank") or 0),
+            head_gate=False, rope_layout="interleaved", rope_scaling=sc)
+    raise ValueError(f"unknown mixer type {kind!r}")
+
+
+def _tudatar_ffn_from_cfg(f: Optional[Dict[str, Any]]
+                          ) -> Optional[MoEFFNSpec]:
+    if not f:
+        return None
+    if f.get("kind", "moe") != "moe":
+        raise ValueError(f"unknown feed-forward kind {f.get('kind')!r}")
+    r = f["router"]
+    E, top = int(r["experts"]), int(r["top"])
+    if not 1 <= top <= E:
+        raise ValueError("router: top must lie between 1 and experts")
+    return MoEFFNSpec(n_experts=E, top_k=top, ff=int(f["expert"]["ff"]),
+                      act="silu_glu", score="sigmoid_all", choice_bias=True,
+                      renorm=True, route_scale=float(r.get("scale", 1.0)))
+
+
+def tanh_layer_specs_from_cfg(layers: List[Dict[str, Any]]
+                              ) -> List[LayerSpec]:
+    """Tudatar: dynamic-tanh norms around a latent attention, a windowed
+    distance-biased attention or a per-channel delta rule, then routed
+    experts."""
+    return [LayerSpec(mixer=_tudatar_mixer_from_cfg(l["type"], l["mixer"]),
+                      ffn=_tudatar_ffn_from_cfg(l.get("mlp")),
+                      form="sandwich_tanh", src=i)
+            for i, l in enumerate(layers)]
+
+
+def mixer_layout(l: LayerSpec) -> Tuple[Dict[str, Tuple[int, int]], int]:
+    """Rows of the ONE input matrix of a layer's mixer: every projection
+    that reads the mixer input, per part in in_sizes order. Every segment
+    starts on a multiple of 8 rows, except that a grouped-query attention's
+    q, k, v stay neighbours. Returns ({name: (offset, size)}, total)."""
     ins: Dict[str, Tuple[int, int]] = {}
     a = 0
     for pre, m in mixer_parts(l.mixer):
@@ -708,6 +797,16 @@ def gated_layout(l: LayerSpec, width: int
             # q, k, v stay neighbours (one conv / one rotation pass)
             a += n if name in ("q", "k") and m.kind == "gqa_attention" \
                 else _pad8(n)
+    return ins, a
+
+
+def gated_layout(l: LayerSpec, width: int
+                 ) -> Tuple[Dict[str, Tuple[int, int]], int]:
+    """Rows of a gated parallel-form layer's ONE input matrix: the mixer's
+    (mixer_layout), then the two residual gates 'rg1' (mixer) and 'rg2'
+    (feed-forward, when there is one), each segment on a multiple of 8
+    rows. Returns ({name: (offset, size)}, total)."""
+    ins, a = mixer_layout(l)
     for name in ("rg1", "rg2") if l.ffn is not None else ("rg1",):
         ins[name] = (a, width)
         a += _pad8(width)
@@ -788,6 +887,9 @@ def hybrid_n_params(width: int, vocab: int, taps: int,
             if l.weights_of is None or active_only:
                 n += _gated_layer_params(width, l, active_only)
             continue
+        if l.form == "sandwich_tanh":
+            n += _tanh_layer_params(width, l, active_only)
+            continue
         n += 4 + width * taps
         if m.kind == "latent_attention":
             n += width * (m.q_size + m.cache_dim + m.heads) + m.kv_rank
@@ -812,6 +914,27 @@ def _sandwich_w_layer_params(width: int, l: LayerSpec,
     elif f is not None:
         e = f.top_k if active_only else f.n_experts
         n += 2 * width + width * f.n_experts + 3 * width * e * f.ff
+    return n
+
+
+def _tanh_layer_params(width: int, l: LayerSpec, active_only: bool) -> int:
+    m, f = l.mixer, l.ffn
+    n = 2 * (2 * width + 1) + width * m.out_size
+    n += width * sum(sz for _, sz in m.in_sizes)
+    if m.kind == "latent_attention":
+        n += m.q_rank + m.kv_rank + m.q_rank * m.q_size
+        n += m.kv_rank * m.heads * (m.dim + m.vdim)
+    elif m.kind == "gqa_attention":
+        n += m.conv_channels + 2 * m.heads
+        n += (m.heads + m.kv_heads) * m.dim
+    else:
+        hd, hv = m.heads * m.dim, m.heads * m.vdim
+        n += m.taps * m.conv_channels + m.heads + m.vdim + hd
+        n += m.decay_rank * hd + m.gate_rank * hv
+    if f is not None:
+        e = f.top_k if active_only else f.n_experts
+        n += 2 * (2 * width + 1) + (width + 1) * f.n_experts
+        n += 3 * width * e * f.ff
     return n
 
 
@@ -999,3 +1122,41 @@ def zevilorn_layer_cfgs(n_layers: int, width: int, *, heads: int = 16,
                      "right": {"width": gru_width or width}}
         cfg_layers.append({"type": typ, "mixer": mixer, "mlp": mlp})
     return cfg_layers
+
+
+def tudatar_layer_cfgs(n_layers: int, width: int, *, heads: int = 16,
+                       kv_heads: int = 4, dim: int = 128, window: int = 1024,
+                       kv_rank: int = 512, rot_dim: int = 64,
+                       q_rank: int = 768, delta_heads: int = 16,
+                       delta_kv_heads: int = 16, delta_dim: int = 128,
+                       rank: int = 64, taps: int = 4, experts: int = 8,
+                       top_k: int = 2, expert_ff: int = 1024
+                       ) -> List[Dict[str, Any]]:
+    """config.json 'layers' entries of a synthetic Tudatar stack for
+    benchmarks: the cycle windowed distance-biased attention / latent
+    attention / per-channel delta rule, every layer with routed experts."""
+    mlp = {"kind": "moe", "expert": {"ff": expert_ff},
+           "router": {"experts": experts, "top": top_k, "scale": 1.25}}
+    out = []
+    for i in range(n_layers):
+        k = i % 3
+        if k == 0:
+            typ = "attention"
+            mixer: Dict[str, Any] = {
+                "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim,
+                "scale": dim ** -0.5, "mask": {"size": window}}
+        elif k == 1:
+            typ = "latent_attention"
+            mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim,
+                     "vdim": dim, "kv_rank": kv_rank, "q_rank": q_rank,
+                     "scale": (dim + rot_dim) ** -0.5,
+                     "rot": {"base": 1e6, "dims": rot_dim,
+                             "scaling": {"factor": 8.0, "original": 4096,
+                                         "fast": 32.0, "slow": 1.0}}}
+        else:
+            typ = "channel_delta"
+            mixer = {"heads": delta_heads, "kv_heads": delta_kv_heads,
+                     "dim": delta_dim, "vdim": delta_dim, "conv": taps,
+                     "decay_rank": rank, "gate_rank": rank}
+        out.append({"type": typ, "mixer": mixer, "mlp": mlp})
+    return out

@@ -48,14 +48,15 @@ class ModelSpec:
     # vocab specials (byte-tokenizer defaults; overridden by a real tokenizer)
     bos_token_id: int = 1
     eos_token_id: int = 2
-    # hybrid stacks (arch "nukopel", "pugozen", "pimodra", "zevilorn"): per-layer mixer/feed-forward specs
-    # (models/hybrid.py). When set, the uniform-layer fields above hold
+    # hybrid stacks (arch "nukopel", "pugozen", "pimodra", "zevilorn",
+    # "tudatar"): per-layer mixer/feed-forward specs (models/hybrid.py). When set, the uniform-layer fields above hold
     # representative maxima only; the Runner's hybrid path reads these.
     layer_specs: Optional[List[Any]] = None
     embed_scale: float = 1.0     # x = embed[token] * embed_scale
     canon_taps: int = 0          # causal per-channel conv on the mixer input
     norm_groups: int = 1         # weighted RMS norms over equal parts of a row
     step_rows: int = 0           # rows of the per-pass residual step table
+    logit_scale: float = 1.0     # logits = head(norm(x)) * logit_scale
     # the config.json "layers" / "loop" entries a looped stack was unrolled
     # from (kept for export)
     source_cfg: Optional[Dict[str, Any]] = None
@@ -522,6 +523,30 @@ def zevilorn_spec(name: str, cfg: Dict[str, Any]) -> ModelSpec:
     return spec
 
 
+def tudatar_spec(name: str, cfg: Dict[str, Any],
+                 shapes: Optional[Dict[str, Any]] = None) -> ModelSpec:
+    """Parse a Tudatar config.json dict: dynamic-tanh norms around latent
+    attention, windowed distance-biased attention or the per-channel gated
+    delta rule, sigmoid-routed experts with a choice bias. `shapes`
+    (checkpoint tensor name -> shape) supplies the low-rank widths that the
+    config does not state."""
+    from .hybrid import complete_from_shapes, tanh_layer_specs_from_cfg
+
+    layers = tanh_layer_specs_from_cfg(cfg["layers"])
+    if shapes:
+        complete_from_shapes(layers, shapes)
+    spec = hybrid_spec(
+        name, int(cfg["vocab"]), int(cfg["width"]), layers,
+        eps=float(cfg["norm"]["eps"]), embed_scale=1.0, canon_taps=0,
+        max_seq_len=int(cfg.get("max_seq_len", 32768)),
+        arch="tudatar", norm_type="tanh", act_type="silu_glu",
+    )
+    spec.n_kv_heads = max(getattr(l.mixer, "kv_heads", 1) for l in layers)
+    spec.logit_scale = float(cfg.get("logit_scale", 1.0))
+    spec.source_cfg = {"layers": cfg["layers"]}
+    return spec
+
+
 def resolve_spec(name: str, model_path: Optional[str] = None) -> ModelSpec:
     """Resolve a model name (preset / alias / HF id / local dir) to a spec.
 
@@ -572,6 +597,12 @@ def spec_from_hf_config(model_path: str, name: Optional[str] = None) -> ModelSpe
     if cfg.get("architecture") == "Zevilorn":
         return zevilorn_spec(
             name or os.path.basename(os.path.normpath(model_path)), cfg)
+    if cfg.get("architecture") == "Tudatar":
+        from .weights import safetensors_shapes
+
+        return tudatar_spec(
+            name or os.path.basename(os.path.normpath(model_path)), cfg,
+            safetensors_shapes(model_path))
     if cfg.get("model_type") == "gpt2" or "n_embd" in cfg:
         spec = _gpt2(
             name or cfg.get("_name_or_path", os.path.basename(model_path)),

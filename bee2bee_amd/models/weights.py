@@ -48,6 +48,9 @@ class LayerWeights:
         "norms", "talk", "act_coef",
         # gated parallel-form layers: the bias of the fused input matrix
         "b_in",
+        # routed experts: a number per expert added to the scores for the
+        # choice; the experts' output matrices side by side [W, E * ff]
+        "moe_choice_bias", "moe_w_down_cat",
     )
 
     def __init__(self) -> None:
@@ -79,9 +82,12 @@ class LayerWeights:
         self.layout = None     # models/hybrid.py fused_layout(layer)
         self.mix = None        # {part prefix: SimpleNamespace of tensors}
         self.norms = None      # 4 x [width] fp32: pre/post mixer, pre/post ffn
+                               # (dynamic tanh: (alpha, weight, bias) each)
         self.talk = None       # [heads, heads] fp32
         self.act_coef = None   # [4] fp32 (PolyNorm a, b, c, e)
         self.b_in = None       # [in_total] (zeros where a part has no bias)
+        self.moe_choice_bias = None   # [E] fp32
+        self.moe_w_down_cat = None    # [width, E * ff]
 
 
 class ModelWeights:
@@ -95,6 +101,10 @@ class ModelWeights:
         self.final_norm_bias: Optional[torch.Tensor] = None
         self.lm_head: Optional[torch.Tensor] = None  # [vocab, hidden]
         self.final_gain: Optional[float] = None  # scalar-gain final norm
+        # dynamic-tanh final norm (alpha, weight, bias), and the same with
+        # the logit scale folded in
+        self.final_tanh: Optional[Tuple] = None
+        self.final_tanh_scaled: Optional[Tuple] = None
         self.step_table: Optional[torch.Tensor] = None  # [passes, hidden] fp32
         self.layers = [LayerWeights() for _ in range(spec.n_layers)]
         # expert-parallel shard: when set, MoE expert tensors hold only
@@ -129,6 +139,8 @@ class ModelWeights:
                 return self._random_init_pimodra(seed)
             if s.arch == "zevilorn":
                 return self._random_init_zevilorn(seed)
+            if s.arch == "tudatar":
+                return self._random_init_tudatar(seed)
             return self._random_init_hybrid(seed)
         lo, hi = layer_range or (0, s.n_layers)
         self.expert_range = expert_range
@@ -232,6 +244,8 @@ class ModelWeights:
                 return self._load_pimodra(model_path)
             if s.arch == "zevilorn":
                 return self._load_zevilorn(model_path)
+            if s.arch == "tudatar":
+                return self._load_tudatar(model_path)
             return self._load_nukopel(model_path)
         if s.arch == "gpt2":
             return self._load_gpt2(model_path, layer_range)
@@ -688,6 +702,251 @@ class ModelWeights:
                 self.layers[i] = self.layers[l.weights_of]
 
 
+    # ---------------------------------- mixer tensors shared by the families
+    # ns: the layer's namespace for this mixer part; put_in(key, name | tensor
+    # [, bias]) places rows of the fused input matrix.
+
+    def _act(self, t: torch.Tensor) -> torch.Tensor:
+        return t.to(self.device, self.dtype).contiguous()
+
+    def _f32(self, t: torch.Tensor) -> torch.Tensor:
+        return t.to(self.device, torch.float32).contiguous()
+
+    def _conv_taps(self, q: str, get) -> torch.Tensor:
+        # checkpoint [channels, taps] -> tap-major [taps, channels]
+        return self._f32(torch.cat([get(q + "q.conv"), get(q + "k.conv"),
+                                    get(q + "v.conv")], dim=0).t())
+
+    def _mix_gqa(self, ns, m, pre: str, q: str, get, put_in) -> None:
+        for n_ in ("q", "k", "v"):
+            put_in(pre + n_, q + n_, m.bias)
+        if m.head_gate:
+            put_in(pre + "g", q + "g")
+        ns.conv_w = self._conv_taps(q, get) if m.taps else None
+        ns.talk = self._f32(get(q + "talk")) if m.score_mix else None
+        ns.q_norm = ns.k_norm = ns.dist = None
+        if m.proj_norm:
+            ns.q_norm = self._f32(get(q + "q.norm"))
+            ns.k_norm = self._f32(get(q + "k.norm"))
+        if m.distance_bias:
+            # [2, heads]: the factor and the rate of the logarithm
+            ns.dist = self._f32(torch.stack([get(q + "r1"), get(q + "r2")]))
+        ns.wo_b = self._act(get(q + "o.b")) if m.bias and m.out_bias else None
+
+    def _mix_latent(self, ns, m, pre: str, q: str, get, put_in) -> None:
+        if m.q_rank:
+            put_in(pre + "dq", q + "dq")
+            ns.q_norm = self._f32(get(q + "dq.norm"))
+            ns.w_uq = self._act(get(q + "uq"))
+        else:
+            put_in(pre + "q", q + "q")
+            ns.q_norm = ns.w_uq = None
+        put_in(pre + "dkv", q + "dkv")
+        if m.head_gate:
+            put_in(pre + "g", q + "g")
+        ns.kv_norm = self._f32(get(q + "dkv.norm"))
+        ns.w_uk = self._act(get(q + "uk").reshape(m.heads, m.dim, m.kv_rank))
+        ns.w_uv = self._act(get(q + "uv").reshape(
+            m.heads, m.vdim, m.kv_rank).transpose(1, 2))
+        ns.sink = self._f32(get(q + "sink")) if m.sink else None
+        ns.wo_b = None
+
+    def _mix_delta(self, ns, m, pre: str, q: str, get, put_in) -> None:
+        put_in(pre + "qkv", torch.cat(
+            [get(q + "q"), get(q + "k"), get(q + "v")], dim=0))
+        ns.conv_w = self._conv_taps(q, get)
+        put_in(pre + "b", get(q + "b"))
+        # decay rate exp(A_log), evaluated once in fp32
+        ns.rate = torch.exp(self._f32(get(q + "A_log")))
+        ns.dt_bias = self._f32(get(q + "dt_bias"))
+        ns.norm = self._f32(get(q + "norm"))
+        if m.channel_decay:
+            put_in(pre + "a", get(q + "a1"))
+            ns.a2 = self._act(get(q + "a2"))
+        else:
+            put_in(pre + "a", get(q + "a"))
+            ns.a2 = None
+        if m.gate_rank:
+            put_in(pre + "g", get(q + "g1"))
+            ns.g2 = self._act(get(q + "g2"))
+        else:
+            put_in(pre + "g", get(q + "g"))
+            ns.g2 = None
+
+    @staticmethod
+    def _latent_shapes(m, W: int) -> Dict[str, tuple]:
+        """{tensor: (shape, init mean, init std)} of a latent attention."""
+        lin, qr = W ** -0.5, max(1, m.q_rank)
+        return {"dq": ((m.q_rank, W), 0.0, lin),
+                "q": ((m.q_size, W), 0.0, lin),
+                "dq.norm": ((m.q_rank,), 1.0, 0.1),
+                "uq": ((m.q_size, qr), 0.0, qr ** -0.5),
+                "dkv": ((m.cache_dim, W), 0.0, lin),
+                "dkv.norm": ((m.kv_rank,), 1.0, 0.1),
+                "uk": ((m.heads * m.dim, m.kv_rank), 0.0, m.kv_rank ** -0.5),
+                "uv": ((m.heads * m.vdim, m.kv_rank), 0.0, m.kv_rank ** -0.5),
+                "sink": ((m.heads,), 0.0, 1.0),
+                "g": ((m.heads, W), 0.0, lin)}
+
+    @staticmethod
+    def _delta_shapes(m, W: int) -> Dict[str, tuple]:
+        """{tensor: (shape, init mean, init std)} of a gated delta rule."""
+        lin = W ** -0.5
+        H, G, D, Dv = m.heads, m.kv_heads, m.dim, m.vdim
+        table = {"q": ((G * D, W), 0.0, lin), "k": ((G * D, W), 0.0, lin),
+                 "v": ((H * Dv, W), 0.0, lin),
+                 "q.conv": ((G * D, m.taps), 0.0, 0.4),
+                 "k.conv": ((G * D, m.taps), 0.0, 0.4),
+                 "v.conv": ((H * Dv, m.taps), 0.0, 0.4),
+                 "b": ((H, W), 0.0, lin), "A_log": ((H,), -1.0, 0.5),
+                 "norm": ((Dv,), 1.0, 0.1)}
+        if m.channel_decay:
+            table.update({"a1": ((m.decay_rank, W), 0.0, lin),
+                          "a2": ((H * D, m.decay_rank), 0.0,
+                                 m.decay_rank ** -0.5),
+                          "dt_bias": ((H * D,), 0.0, 0.5)})
+        else:
+            table.update({"a": ((H, W), 0.0, lin), "dt_bias": ((H,), 0.0, 0.5)})
+        if m.gate_rank:
+            table.update({"g1": ((m.gate_rank, W), 0.0, lin),
+                          "g2": ((H * Dv, m.gate_rank), 0.0,
+                                 m.gate_rank ** -0.5)})
+        else:
+            table["g"] = ((H * Dv, W), 0.0, lin)
+        return table
+
+    # ------------------------------------------------ dynamic-tanh stacks
+
+    @torch.no_grad()
+    def _load_tudatar(self, model_path: str) -> "ModelWeights":
+        """Tudatar safetensors: 'embed', 'head', 'final.norm' and per layer
+        'l<i>.norm1|norm1b|norm2|norm2b', 'l<i>.mix.*',
+        'l<i>.mlp.router|correction|e<k>.gate|up|down'. A norm is a weight
+        plus '.b' and the scalar '.alpha'. Linear weights [out, in]."""
+        tensors = dict(iter_safetensors(model_path))
+        self._assemble_tudatar(lambda name: tensors.pop(name))
+        return self
+
+    @torch.no_grad()
+    def _random_init_tudatar(self, seed: int) -> "ModelWeights":
+        import zlib
+
+        def get(name: str) -> torch.Tensor:
+            tseed = (seed * 1000003 + zlib.crc32(name.encode())) % (2**31)
+            gen = torch.Generator(device=self.device).manual_seed(tseed)
+            shape, mean, std = self._tudatar_shape(name)
+            t = torch.randn(tuple(shape), generator=gen, dtype=torch.float32,
+                            device=self.device)
+            t = mean + std * t
+            return (t.abs() if name.endswith(".r2") else t).bfloat16()
+
+        self._assemble_tudatar(get)
+        return self
+
+    def _tudatar_shape(self, name: str):
+        """(shape, init mean, init std) of a checkpoint tensor."""
+        s = self.spec
+        W, V = s.hidden_size, s.vocab_size
+        lin = W ** -0.5
+        if name == "embed":
+            return (V, W), 0.0, 1.0
+        if name == "head":
+            return (V, W), 0.0, lin
+        head, rest = name.split(".", 1)
+        if head == "final" or rest.startswith("norm"):
+            if rest.endswith(".alpha"):
+                return (), 0.6, 0.1
+            return (W,), (0.0 if rest.endswith(".b") else 1.0), 0.1
+        l = s.layer_specs[int(head[1:])]
+        m, f = l.mixer, l.ffn
+        if rest.startswith("mlp."):
+            rest = rest[len("mlp."):]
+            if rest == "router":
+                return (f.n_experts, W), 0.0, lin
+            if rest == "correction":
+                return (f.n_experts,), 0.0, 0.1
+            if rest.endswith(".down"):
+                return (W, f.ff), 0.0, f.ff ** -0.5
+            return (f.ff, W), 0.0, lin
+        rest = rest[len("mix."):]
+        if rest == "o":
+            return (W, m.out_size), 0.0, m.out_size ** -0.5
+        if m.kind == "latent_attention":
+            return self._latent_shapes(m, W)[rest]
+        if m.kind == "delta":
+            return self._delta_shapes(m, W)[rest]
+        sizes = dict(m.in_sizes)
+        if rest in ("r1", "r2"):
+            return (m.heads,), 0.5, 0.2
+        if rest.endswith(".norm"):
+            return (sizes[rest[:-5]],), 1.0, 0.1
+        if rest.endswith(".b"):
+            return (sizes[rest[:-2]],), 0.0, 0.1
+        return (sizes[rest], W), 0.0, lin
+
+    def _assemble_tudatar(self, get) -> None:
+        """Engine layout of a dynamic-tanh stack: per layer ONE input matrix
+        for the mixer (models/hybrid.py mixer_layout; a bias vector where
+        the mixer has biases), the norms as (alpha, weight, bias) with a
+        host-side alpha and fp32 vectors, router and choice bias in fp32,
+        expert input matrices [E, 2ff, W], and the expert output matrices
+        side by side as ONE [W, E * ff] matrix (so a step with few tokens
+        sums its experts inside one product); `moe_w_down` is its
+        per-expert view [E, W, ff]. The logit scale is folded into the
+        final norm's weight and bias."""
+        from types import SimpleNamespace
+
+        from .hybrid import mixer_layout
+
+        s = self.spec
+        W = s.hidden_size
+
+        def norm(name: str):
+            return (float(get(name + ".alpha").float()),
+                    self._f32(get(name)), self._f32(get(name + ".b")))
+
+        self.embed = self._act(get("embed"))
+        self.lm_head = self._act(get("head"))
+        a, w, b = self.final_tanh = norm("final.norm")
+        self.final_tanh_scaled = (a, w * s.logit_scale, b * s.logit_scale)
+        for i, l in enumerate(s.layer_specs):
+            lw, p, m, f = self.layers[i], f"l{i}.", l.mixer, l.ffn
+            ins, n_in = mixer_layout(l)
+            lw.layout = (ins, n_in)
+            names = ("norm1", "norm1b") + (("norm2", "norm2b") if f else ())
+            lw.norms = [norm(p + n) for n in names]
+            w_in = torch.zeros(n_in, W, device=self.device, dtype=self.dtype)
+            b_in = torch.zeros(n_in, device=self.device, dtype=self.dtype)
+
+            def put_in(key: str, t, bias: bool = False) -> None:
+                off, n = ins[key]
+                name, t = (t, get(t)) if isinstance(t, str) else (key, t)
+                assert t.shape == (n, W), (name, tuple(t.shape), n)
+                w_in[off : off + n] = t.to(self.device, self.dtype)
+                if bias:
+                    b_in[off : off + n] = get(name + ".b").to(self.device,
+                                                              self.dtype)
+
+            ns = SimpleNamespace()
+            lw.mix = {"": ns}
+            mix = {"gqa_attention": self._mix_gqa, "delta": self._mix_delta,
+                   "latent_attention": self._mix_latent}[m.kind]
+            mix(ns, m, "", p + "mix.", get, put_in)
+            ns.wo = self._act(get(p + "mix.o"))
+            lw.w_in = w_in
+            lw.b_in = b_in if getattr(m, "bias", False) else None
+            if f is None:
+                continue
+            lw.moe_gate = self._f32(get(p + "mlp.router"))
+            lw.moe_choice_bias = self._f32(get(p + "mlp.correction"))
+            lw.moe_w_gate_up = self._act(torch.stack([
+                torch.cat([get(f"{p}mlp.e{e}.gate"), get(f"{p}mlp.e{e}.up")])
+                for e in range(f.n_experts)]))
+            lw.moe_w_down_cat = self._act(torch.cat([
+                get(f"{p}mlp.e{e}.down") for e in range(f.n_experts)], dim=1))
+            lw.moe_w_down = lw.moe_w_down_cat.view(
+                W, f.n_experts, f.ff).permute(1, 0, 2)
+
     # --------------------------------------------- gated parallel-form stacks
 
     @torch.no_grad()
@@ -758,20 +1017,7 @@ class ModelWeights:
             return (W,), 0.0, 0.1
         sizes = dict(m.in_sizes)
         if m.kind == "latent_attention":
-            table = {"dq": ((m.q_rank, W), 0.0, lin),
-                     "q": ((m.q_size, W), 0.0, lin),
-                     "dq.norm": ((m.q_rank,), 1.0, 0.1),
-                     "uq": ((m.q_size, max(1, m.q_rank)), 0.0,
-                            max(1, m.q_rank) ** -0.5),
-                     "dkv": ((m.cache_dim, W), 0.0, lin),
-                     "dkv.norm": ((m.kv_rank,), 1.0, 0.1),
-                     "uk": ((m.heads * m.dim, m.kv_rank), 0.0,
-                            m.kv_rank ** -0.5),
-                     "uv": ((m.heads * m.vdim, m.kv_rank), 0.0,
-                            m.kv_rank ** -0.5),
-                     "sink": ((m.heads,), 0.0, 1.0),
-                     "g": ((m.heads, W), 0.0, lin)}
-            return table[rest]
+            return self._latent_shapes(m, W)[rest]
         if m.kind == "gqa_attention" and rest == "talk":
             return (m.heads, m.heads), 0.0, 0.1
         if rest.endswith(".conv"):
@@ -829,33 +1075,9 @@ class ModelWeights:
                 q = p + "mix." + pre
                 ns = lw.mix[pre] = SimpleNamespace()
                 if m.kind == "gqa_attention":
-                    for n_ in ("q", "k", "v"):
-                        put_in(pre + n_, q + n_, m.bias)
-                    if m.head_gate:
-                        put_in(pre + "g", q + "g")
-                    # checkpoint [channels, taps] -> tap-major [taps, channels]
-                    ns.conv_w = f32(torch.cat(
-                        [get(q + "q.conv"), get(q + "k.conv"),
-                         get(q + "v.conv")], dim=0).t()) if m.taps else None
-                    ns.talk = f32(get(q + "talk")) if m.score_mix else None
-                    ns.wo_b = act(get(q + "o.b")) if m.bias else None
+                    self._mix_gqa(ns, m, pre, q, get, put_in)
                 elif m.kind == "latent_attention":
-                    if m.q_rank:
-                        put_in(pre + "dq", q + "dq")
-                        ns.q_norm = f32(get(q + "dq.norm"))
-                        ns.w_uq = act(get(q + "uq"))
-                    else:
-                        put_in(pre + "q", q + "q")
-                        ns.q_norm = ns.w_uq = None
-                    put_in(pre + "dkv", q + "dkv")
-                    put_in(pre + "g", q + "g")
-                    ns.kv_norm = f32(get(q + "dkv.norm"))
-                    ns.w_uk = act(get(q + "uk").reshape(
-                        m.heads, m.dim, m.kv_rank))
-                    ns.w_uv = act(get(q + "uv").reshape(
-                        m.heads, m.vdim, m.kv_rank).transpose(1, 2))
-                    ns.sink = f32(get(q + "sink")) if m.sink else None
-                    ns.wo_b = None
+                    self._mix_latent(ns, m, pre, q, get, put_in)
                 else:
                     put_in(pre + "z", q + "z", True)
                     put_in(pre + "x", q + "x", True)
@@ -941,28 +1163,7 @@ class ModelWeights:
             return {"q": ((H * D, W), 0.0, lin), "k": ((G * D, W), 0.0, lin),
                     "q.norm": ((D,), 1.0, 0.1), "k.norm": ((D,), 1.0, 0.1),
                     "temp": ((H,), 1.0, 0.2), "sink": ((H,), 0.0, 1.0)}[rest]
-        G = m.kv_heads
-        table = {"q": ((G * D, W), 0.0, lin), "k": ((G * D, W), 0.0, lin),
-                 "v": ((H * Dv, W), 0.0, lin),
-                 "q.conv": ((G * D, m.taps), 0.0, 0.4),
-                 "k.conv": ((G * D, m.taps), 0.0, 0.4),
-                 "v.conv": ((H * Dv, m.taps), 0.0, 0.4),
-                 "b": ((H, W), 0.0, lin), "A_log": ((H,), -1.0, 0.5),
-                 "norm": ((Dv,), 1.0, 0.1)}
-        if m.channel_decay:
-            table.update({"a1": ((m.decay_rank, W), 0.0, lin),
-                          "a2": ((H * D, m.decay_rank), 0.0,
-                                 m.decay_rank ** -0.5),
-                          "dt_bias": ((H * D,), 0.0, 0.5)})
-        else:
-            table.update({"a": ((H, W), 0.0, lin), "dt_bias": ((H,), 0.0, 0.5)})
-        if m.gate_rank:
-            table.update({"g1": ((m.gate_rank, W), 0.0, lin),
-                          "g2": ((H * Dv, m.gate_rank), 0.0,
-                                 m.gate_rank ** -0.5)})
-        else:
-            table["g"] = ((H * Dv, W), 0.0, lin)
-        return table[rest]
+        return self._delta_shapes(m, W)[rest]
 
     def _assemble_pugozen(self, get) -> None:
         """Engine layout of a parallel-form stack: per layer ONE input GEMM
@@ -1022,29 +1223,7 @@ class ModelWeights:
                     # score = (q . k) * scale * temp_h, folded into q
                     ns.q_mult = ns.temp * m.scale
                 else:
-                    put_in(pre + "qkv", torch.cat(
-                        [get(q + "q"), get(q + "k"), get(q + "v")], dim=0))
-                    # checkpoint [channels, taps] -> tap-major [taps, channels]
-                    ns.conv_w = f32(torch.cat(
-                        [get(q + "q.conv"), get(q + "k.conv"),
-                         get(q + "v.conv")], dim=0).t())
-                    put_in(pre + "b", get(q + "b"))
-                    # decay rate exp(A_log), evaluated once in fp32
-                    ns.rate = torch.exp(f32(get(q + "A_log")))
-                    ns.dt_bias = f32(get(q + "dt_bias"))
-                    ns.norm = f32(get(q + "norm"))
-                    if m.channel_decay:
-                        put_in(pre + "a", get(q + "a1"))
-                        ns.a2 = act(get(q + "a2"))
-                    else:
-                        put_in(pre + "a", get(q + "a"))
-                        ns.a2 = None
-                    if m.gate_rank:
-                        put_in(pre + "g", get(q + "g1"))
-                        ns.g2 = act(get(q + "g2"))
-                    else:
-                        put_in(pre + "g", get(q + "g"))
-                        ns.g2 = None
+                    self._mix_delta(ns, m, pre, q, get, put_in)
                 off, n = outs[pre + "o"]
                 w_out[:, off : off + n] = get(q + "o").to(dev, dt)
             if l.ffn is not None:
@@ -1219,6 +1398,87 @@ def _save_zevilorn(weights: "ModelWeights", out_dir: str, tensors, cpu) -> None:
     save_file(tensors, os.path.join(out_dir, "model.safetensors"))
     with open(os.path.join(out_dir, "config.json"), "w") as fh:
         json.dump(zevilorn_config(s), fh, indent=1)
+
+
+def tudatar_config(spec: ModelSpec) -> Dict:
+    """The config.json dict of a Tudatar spec (inverse of tudatar_spec): the
+    layer entries are kept as they were parsed."""
+    return {"architecture": "Tudatar", "vocab": spec.vocab_size,
+            "width": spec.hidden_size, "max_seq_len": spec.max_seq_len,
+            "norm": {"eps": spec.rms_eps}, "logit_scale": spec.logit_scale,
+            "layers": (spec.source_cfg or {}).get("layers", [])}
+
+
+def _save_tudatar(weights: "ModelWeights", out_dir: str, tensors, cpu) -> None:
+    from safetensors.torch import save_file
+
+    s = weights.spec
+
+    def put(name: str, t: torch.Tensor) -> None:
+        tensors[name] = cpu(t).to(torch.bfloat16)
+
+    def norm(name: str, n) -> None:
+        put(name + ".alpha", torch.tensor(n[0]))
+        put(name, n[1])
+        put(name + ".b", n[2])
+
+    put("embed", weights.embed)
+    put("head", weights.lm_head)
+    norm("final.norm", weights.final_tanh)
+    for i, l in enumerate(s.layer_specs):
+        lw, p, m, f = weights.layers[i], f"l{i}.", l.mixer, l.ffn
+        ins, ns, q = lw.layout[0], lw.mix[""], f"l{i}.mix."
+        for n_, t in zip(("norm1", "norm1b", "norm2", "norm2b"), lw.norms):
+            norm(p + n_, t)
+
+        def rows(key: str, name: str) -> None:
+            off, n = ins[key]
+            put(name, lw.w_in[off : off + n])
+
+        put(q + "o", ns.wo)
+        if m.kind == "gqa_attention":
+            for n_ in ("q", "k", "v"):
+                rows(n_, q + n_)
+                off, n = ins[n_]
+                put(q + n_ + ".b", lw.b_in[off : off + n])
+            put(q + "q.norm", ns.q_norm)
+            put(q + "k.norm", ns.k_norm)
+            put(q + "r1", ns.dist[0])
+            put(q + "r2", ns.dist[1])
+        elif m.kind == "latent_attention":
+            rows("dq", q + "dq")
+            put(q + "dq.norm", ns.q_norm)
+            put(q + "uq", ns.w_uq)
+            rows("dkv", q + "dkv")
+            put(q + "dkv.norm", ns.kv_norm)
+            put(q + "uk", ns.w_uk.reshape(m.heads * m.dim, m.kv_rank))
+            put(q + "uv", ns.w_uv.transpose(1, 2).reshape(
+                m.heads * m.vdim, m.kv_rank))
+        else:
+            nq, nv = m.kv_heads * m.dim, m.heads * m.vdim
+            off, at = ins["qkv"][0], 0
+            for n_, sz in (("q", nq), ("k", nq), ("v", nv)):
+                put(q + n_, lw.w_in[off + at : off + at + sz])
+                put(q + n_ + ".conv", ns.conv_w[:, at : at + sz].t())
+                at += sz
+            rows("b", q + "b")
+            put(q + "A_log", torch.log(ns.rate))
+            put(q + "dt_bias", ns.dt_bias)
+            put(q + "norm", ns.norm)
+            rows("a", q + "a1")
+            put(q + "a2", ns.a2)
+            rows("g", q + "g1")
+            put(q + "g2", ns.g2)
+        if f is not None:
+            put(p + "mlp.router", lw.moe_gate)
+            put(p + "mlp.correction", lw.moe_choice_bias)
+            for e in range(f.n_experts):
+                put(f"{p}mlp.e{e}.gate", lw.moe_w_gate_up[e, : f.ff])
+                put(f"{p}mlp.e{e}.up", lw.moe_w_gate_up[e, f.ff :])
+                put(f"{p}mlp.e{e}.down", lw.moe_w_down[e])
+    save_file(tensors, os.path.join(out_dir, "model.safetensors"))
+    with open(os.path.join(out_dir, "config.json"), "w") as fh:
+        json.dump(tudatar_config(s), fh, indent=1)
 
 
 def safetensors_shapes(model_path: str) -> Dict[str, Tuple[int, ...]]:
@@ -1516,6 +1776,8 @@ def save_hf(weights: ModelWeights, out_dir: str) -> None:
             _save_pimodra(weights, out_dir, tensors, cpu)
         elif s.arch == "zevilorn":
             _save_zevilorn(weights, out_dir, tensors, cpu)
+        elif s.arch == "tudatar":
+            _save_tudatar(weights, out_dir, tensors, cpu)
         else:
             _save_nukopel(weights, out_dir, tensors, cpu)
         return

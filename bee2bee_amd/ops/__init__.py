@@ -274,14 +274,15 @@ def canon_conv(h, w, state, state_slots, cu_seqlens, seq_idx, positions):
 
 def latent_rope_store(q_rot, kv, kv_norm, eps: float, kv_rank: int,
                       rope_dims: int, positions, cos, sin, cache,
-                      slot_mapping) -> None:
+                      slot_mapping, interleaved: bool = False) -> None:
     if _use_hip(kv):
         require_hip().latent_rope_store(q_rot, kv, kv_norm, eps, kv_rank,
                                         rope_dims, positions, cos, sin, cache,
-                                        slot_mapping)
+                                        slot_mapping, interleaved)
         return
     reference.latent_rope_store(q_rot, kv, kv_norm, eps, kv_rank, rope_dims,
-                                positions, cos, sin, cache, slot_mapping)
+                                positions, cos, sin, cache, slot_mapping,
+                                interleaved)
 
 
 def latent_attn(q_abs, q_rot, gate, cache, block_table, positions, seq_idx,
@@ -290,7 +291,7 @@ def latent_attn(q_abs, q_rot, gate, cache, block_table, positions, seq_idx,
     """max_qlen: longest chunk in the batch (host int); 1 selects the
     decode kernel, larger the query-tiled prefill kernel. window 0: every
     earlier position; sink fp32 [heads]: a logit per head in the softmax
-    denominator."""
+    denominator; gate None: no output gate."""
     if _use_hip(q_abs):
         return require_hip().latent_attn(q_abs, q_rot, gate, cache,
                                          block_table, positions, seq_idx,
@@ -483,7 +484,9 @@ def silu_glu(gate_up):
 
 
 def group_topk_gate(logits, top_k: int, n_groups: int, keep_groups: int,
-                    score: str = "softmax", group_top: int = 1):
+                    score: str = "softmax", group_top: int = 1,
+                    choice_bias=None, renorm: bool = False,
+                    route_scale: float = 1.0):
     """One kernel on the GPU (a thread per token, scores in LDS) while the
     experts of a workgroup's tokens fit; torch ops otherwise and on the
     CPU."""
@@ -491,10 +494,12 @@ def group_topk_gate(logits, top_k: int, n_groups: int, keep_groups: int,
     if _use_hip(logits) and (E + n_groups) * 256 <= 64 * 1024:
         w, idx = require_hip().group_topk_gate(
             logits.float().contiguous(), top_k, n_groups, keep_groups,
-            score == "sigmoid", group_top)
+            score == "sigmoid", group_top, choice_bias, renorm,
+            float(route_scale))
         return w, idx
     return reference.group_topk_gate(logits, top_k, n_groups, keep_groups,
-                                     score, group_top)
+                                     score, group_top, choice_bias, renorm,
+                                     route_scale)
 
 
 # ------------------------------------------- gated parallel-form stacks
@@ -517,8 +522,10 @@ def rope_store(q, k, v, q_out, rope_dims: int, interleaved: bool, positions,
 
 def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
              cu_seqlens, softcap: float, talk, sink, head_gate, window: int,
-             out, max_qlen: int = 0) -> None:
-    """max_qlen: longest chunk of the step (host int). Without a cap and a
+             out, max_qlen: int = 0, dist=None) -> None:
+    """max_qlen: longest chunk of the step (host int). dist fp32 [2, H]: a
+    logarithmic distance bias on the scores (not together with a cap or a
+    score mix). Without a cap and a
     score mix the step runs on the sink-attention kernels; with them, on
     the score-mixing kernels. Both take bf16 prompt portions with head size
     64/128 to the matrix cores."""
@@ -526,8 +533,12 @@ def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
         if talk is None and not softcap:
             require_hip().sink_attn(q, k_cache, v_cache, block_table,
                                     positions, seq_idx, cu_seqlens, sink,
-                                    window, out, 1.0, max_qlen, head_gate)
+                                    window, out, 1.0, max_qlen, head_gate,
+                                    dist)
         else:
+            if dist is not None:
+                raise ValueError("a distance bias does not combine with a "
+                                 "score cap or mix")
             if talk is None:    # a cap alone: mix with the identity
                 talk = torch.eye(q.shape[1], dtype=torch.float32,
                                  device=q.device)
@@ -537,7 +548,8 @@ def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
                                            head_gate, window, out, max_qlen)
         return
     reference.gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
-                       cu_seqlens, softcap, talk, sink, head_gate, window, out)
+                       cu_seqlens, softcap, talk, sink, head_gate, window, out,
+                       dist)
 
 
 def min_gru(z, x, g, state, state_slots, cu_seqlens, positions, out,
@@ -576,3 +588,36 @@ def gelu_erf(x):
     if _use_hip(x):
         return require_hip().gelu_erf(x)
     return reference.gelu_erf(x)
+
+
+# --------------------------------------------------- dynamic-tanh stacks
+# (ops/reference.py documents shapes and formulas)
+
+
+def add_tanh_norm(resid, y, post, pre, out_dtype):
+    """resid(fp32) += tanh(a y) w + b in place (post = (a, w, b), when y is
+    given); -> the same form of resid with pre (None when pre is None). One
+    element-wise pass on the GPU."""
+    if _use_hip(resid):
+        pa, pw, pb = post if post is not None else (0.0, None, None)
+        na, nw, nb = pre if pre is not None else (0.0, None, None)
+        return require_hip().add_tanh_norm(resid, y, pa, pw, pb, na, nw, nb,
+                                           out_dtype)
+    return reference.add_tanh_norm(resid, y, post, pre, out_dtype)
+
+
+def proj_norm_store(q, k, v, q_norm, k_norm, v_unit: bool, eps: float,
+                    q_mult: float, k_cache, v_cache, slot_mapping) -> None:
+    if _use_hip(q):
+        require_hip().proj_norm_store(q, k, v, q_norm, k_norm, v_unit, eps,
+                                      float(q_mult), k_cache, v_cache,
+                                      slot_mapping)
+        return
+    reference.proj_norm_store(q, k, v, q_norm, k_norm, v_unit, eps, q_mult,
+                              k_cache, v_cache, slot_mapping)
+
+
+def routed_silu_glu(gu, weights, idx):
+    if _use_hip(gu):
+        return require_hip().routed_silu_glu(gu, weights, idx)
+    return reference.routed_silu_glu(gu, weights, idx)

@@ -141,7 +141,9 @@ __global__ __launch_bounds__(64) void attn_prefill_basic(
 // and is multiplied by out_scale. window > 0: the row at absolute position
 // p sees keys p - window < j <= p, and key tiles wholly before the tile's
 // first window are skipped. head_gate (optional, bf16 [tokens, nq] with row
-// stride s_g): head h's output times sigmoid(head_gate[t, h]).
+// stride s_g): head h's output times sigmoid(head_gate[t, h]). DIST:
+// dist [2, nq] = (a, b), a_h ln(1 + b_h d) is taken off a score whose key
+// lies d positions back.
 //
 // MODE 1 / MODE 2 split the kernel around a score buffer, for attention
 // whose scores are mixed across heads before the softmax: MODE 1 stops
@@ -153,7 +155,8 @@ __global__ __launch_bounds__(64) void attn_prefill_basic(
 // query rows [qt0 * 64, qt0 * 64 + qt_rows) of every chunk; entry `col` of
 // a row is key kv_lo + col, kv_lo being the first key the row's 64-query
 // tile visits. blockIdx.x counts tiles from qt0.
-template <int HD, bool PAGED, typename KVT, bool HILO = false, int MODE = 0>
+template <int HD, bool PAGED, typename KVT, bool HILO = false, int MODE = 0,
+          bool DIST = false>
 __global__ __launch_bounds__(256) void attn_prefill_mfma(
     const unsigned short* __restrict__ q,
     const KVT* __restrict__ k,  // PAGED: k_cache [nb,nkv,bs,hd]
@@ -166,7 +169,8 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
     float scale, const float* __restrict__ sink, float out_scale, long s_o,
     int window = 0, const unsigned short* __restrict__ head_gate = nullptr,
     long s_g = 0, float* __restrict__ score_buf = nullptr, int qt0 = 0,
-    int qt_rows = 0, long ctx = 0, float softcap = 0.f) {
+    int qt_rows = 0, long ctx = 0, float softcap = 0.f,
+    const float* __restrict__ dist = nullptr) {
     constexpr int KSTEPS = HD / 32;
     const int seq = blockIdx.z;
     const int h = blockIdx.y;
@@ -229,6 +233,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
 #pragma unroll
     for (int nb = 0; nb < HD / 16; ++nb) o_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 
+    const float da = DIST ? dist[h] : 0.f, db = DIST ? dist[nq + h] : 0.f;
     // causal: keys up to the last absolute q position of this tile
     const int kv_end = min(L, hist + q0 + PF_TM);
     // window: the tile's first row is the one that reaches back farthest
@@ -330,6 +335,11 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
             for (int r = 0; r < 4; ++r) {
                 const int qrow = q0 + wid * PF_QROWS + lg * 4 + r;
                 const int key = kb + f * 16 + li;
+                if (DIST) {
+                    // keys ahead of the row are masked below
+                    const float d = (float)max(hist + qrow - key, 0);
+                    sfrag[f][r] -= da * __logf(1.f + db * d);
+                }
                 if (key > hist + qrow || qrow >= QL || key >= kv_end ||
                     (window > 0 && key <= hist + qrow - window))
                     sfrag[f][r] = -1e30f;
@@ -519,32 +529,31 @@ extern "C" void launch_attn_prefill_paged(
 // weights (bf16 hi+lo pair), an optional per-head sink logit, an output
 // scale and a strided output (a column slice of a wider buffer). bf16,
 // head size 64 or 128 (returns nonzero otherwise); scale is applied by the
-// caller (folded into q). window 0: causal without a window; head_gate
-// optional (see the kernel).
+// caller (folded into q). window 0: causal without a window; head_gate and
+// dist optional (see the kernel).
 extern "C" int launch_attn_prefill_paged_sink(
     const unsigned short* q, long s_q, const unsigned short* k_cache,
     const unsigned short* v_cache, const int* cu, const int* block_table,
     const int* seq_lens, unsigned short* out, long s_o, int nseq, int nq,
     int nkv, int hd, int W, int bs, int max_qlen, const float* sink,
     float out_scale, int window, const unsigned short* head_gate, long s_g,
-    hipStream_t stream) {
+    const float* dist, hipStream_t stream) {
     if (hd != 64 && hd != 128) return 1;
     if (nseq == 0 || max_qlen == 0) return 0;
     const int tiles = (max_qlen + PF_TM - 1) / PF_TM;
     dim3 grid(tiles, nq, nseq);
     const int smem = prefill_mfma_smem(hd, 1);
-    if (hd == 128)
-        hipLaunchKernelGGL(
-            (attn_prefill_mfma<128, true, unsigned short, true>), grid,
-            dim3(256), smem, stream, q, k_cache, v_cache, cu, block_table,
-            seq_lens, out, nq, nkv, s_q, 0, 0, W, bs, 1.f, sink, out_scale,
-            s_o, window, head_gate, s_g);
-    else
-        hipLaunchKernelGGL(
-            (attn_prefill_mfma<64, true, unsigned short, true>), grid,
-            dim3(256), smem, stream, q, k_cache, v_cache, cu, block_table,
-            seq_lens, out, nq, nkv, s_q, 0, 0, W, bs, 1.f, sink, out_scale,
-            s_o, window, head_gate, s_g);
+#define PS_LAUNCH(HDV, DI)                                                    \
+    hipLaunchKernelGGL(                                                       \
+        (attn_prefill_mfma<HDV, true, unsigned short, true, 0, DI>), grid,    \
+        dim3(256), smem, stream, q, k_cache, v_cache, cu, block_table,        \
+        seq_lens, out, nq, nkv, s_q, 0, 0, W, bs, 1.f, sink, out_scale, s_o,  \
+        window, head_gate, s_g, nullptr, 0, 0, 0, 0.f, dist)
+    if (hd == 128 && dist) PS_LAUNCH(128, true);
+    else if (hd == 128) PS_LAUNCH(128, false);
+    else if (dist) PS_LAUNCH(64, true);
+    else PS_LAUNCH(64, false);
+#undef PS_LAUNCH
     return 0;
 }
 

@@ -396,18 +396,22 @@ min_gru_scan_kernel(const int* __restrict__ cu,
 }
 
 // ------------------------------------------------ group-limited routing
-// One thread per token; its E scores (and group scores) live in LDS at
-// stride blockDim, so neighbouring threads never share a bank. scores =
-// sigmoid(logit) or softmax over all experts; a group's score is the sum of
-// its group_top largest scores; experts outside the best `keep` groups
-// cannot be chosen; the top_k best remaining scores are the weights, as they
-// are, in descending order (ties: the lower index first).
+// One thread per token; its E choice scores (and group scores) live in LDS
+// at stride blockDim, so neighbouring threads never share a bank. scores =
+// sigmoid(logit) or softmax over all experts; choice scores add a number per
+// expert when choice_bias is given. A group's score is the sum of its
+// group_top largest choice scores; experts outside the best `keep` groups
+// cannot be chosen; the top_k best remaining are chosen (ties: the lower
+// index first). Weights: the chosen experts' scores WITHOUT the bias,
+// divided by their sum (+ 1e-20) when renorm, times route_scale.
 constexpr int GT_THREADS = 64;
 __global__ void __launch_bounds__(GT_THREADS)
 group_topk_gate_kernel(const float* __restrict__ logits,
+                       const float* __restrict__ choice_bias,
                        float* __restrict__ w_out, int* __restrict__ idx_out,
                        long T, int E, int top_k, int n_groups, int keep,
-                       int group_top, int sigmoid) {
+                       int group_top, int sigmoid, int renorm,
+                       float route_scale) {
     extern __shared__ __attribute__((aligned(16))) float gt_s[];
     const long t = (long)blockIdx.x * GT_THREADS + threadIdx.x;
     if (t >= T) return;                    // no workgroup barrier below
@@ -427,9 +431,13 @@ group_topk_gate_kernel(const float* __restrict__ logits,
         }
         for (int e = 0; e < E; ++e) sc[e * st] /= sum;
     }
+    if (choice_bias)
+        for (int e = 0; e < E; ++e) sc[e * st] += choice_bias[e];
     const int gs = E / n_groups;
     const bool limited = n_groups > 1 && keep < n_groups;
+    unsigned long long kept = ~0ull;       // bit g: group g (n_groups <= 64)
     if (limited) {
+        kept = 0;
         const int gt = min(max(group_top, 1), gs);
         for (int g = 0; g < n_groups; ++g) {
             // sum of the gt largest: each pass takes the largest score that
@@ -437,8 +445,8 @@ group_topk_gate_kernel(const float* __restrict__ logits,
             float total = 0.f, last = INFINITY;
             int last_i = -1;
             for (int it = 0; it < gt; ++it) {
-                float best = -1.f;
-                int bi = -1;
+                float best = -INFINITY;
+                int bi = 0;
                 for (int j = 0; j < gs; ++j) {
                     const float x = sc[(g * gs + j) * st];
                     const bool open = x < last || (x == last && j > last_i);
@@ -451,26 +459,39 @@ group_topk_gate_kernel(const float* __restrict__ logits,
             gsc[g * st] = total;
         }
         for (int it = 0; it < keep; ++it) {
-            float best = -1.f;
-            int bg = 0;
+            float best = -INFINITY;
+            int bg = -1;
             for (int g = 0; g < n_groups; ++g) {
                 const float x = gsc[g * st];
-                if (x > best) { best = x; bg = g; }
+                if (!((kept >> g) & 1) && (bg < 0 || x > best)) {
+                    best = x;
+                    bg = g;
+                }
             }
-            gsc[bg * st] = -2.f;           // kept
+            kept |= 1ull << bg;
         }
     }
+    float total = 0.f;
     for (int it = 0; it < top_k; ++it) {
-        float best = -1.f;
-        int be = 0;
+        float best = -INFINITY;
+        int be = -1;
         for (int e = 0; e < E; ++e) {
-            if (limited && gsc[(e / gs) * st] != -2.f) continue;
+            if (limited && !((kept >> (e / gs)) & 1)) continue;
             const float x = sc[e * st];
             if (x > best) { best = x; be = e; }
         }
-        w_out[t * top_k + it] = best;
+        if (be < 0) be = 0;                // only when scores are not numbers
+        float w = best;
+        if (choice_bias) w = sigmoid ? sigmoid_f(z[be])
+                                     : best - choice_bias[be];
+        w_out[t * top_k + it] = w;
         idx_out[t * top_k + it] = be;
-        sc[be * st] = -1.f;                // taken
+        total += w;
+        sc[be * st] = -INFINITY;           // taken
+    }
+    if (renorm || route_scale != 1.f) {
+        const float r = renorm ? route_scale / (total + 1e-20f) : route_scale;
+        for (int it = 0; it < top_k; ++it) w_out[t * top_k + it] *= r;
     }
 }
 
@@ -614,16 +635,18 @@ extern "C" void launch_min_gru(const void* z, long zs, const void* x, long xs,
 }
 
 // Returns nonzero when the scores of a workgroup's tokens do not fit LDS.
-extern "C" int launch_group_topk_gate(const float* logits, float* w_out,
+extern "C" int launch_group_topk_gate(const float* logits,
+                                      const float* choice_bias, float* w_out,
                                       int* idx_out, long T, int E, int top_k,
                                       int n_groups, int keep, int group_top,
-                                      int sigmoid, hipStream_t s) {
+                                      int sigmoid, int renorm,
+                                      float route_scale, hipStream_t s) {
     const size_t smem = (size_t)(E + n_groups) * GT_THREADS * sizeof(float);
     if (smem > 64 * 1024) return 1;
     if (T == 0) return 0;
     const unsigned grid = (unsigned)((T + GT_THREADS - 1) / GT_THREADS);
     group_topk_gate_kernel<<<grid, GT_THREADS, smem, s>>>(
-        logits, w_out, idx_out, T, E, top_k, n_groups, keep, group_top,
-        sigmoid);
+        logits, choice_bias, w_out, idx_out, T, E, top_k, n_groups, keep,
+        group_top, sigmoid, renorm, route_scale);
     return 0;
 }

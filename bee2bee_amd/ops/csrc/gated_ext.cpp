@@ -38,8 +38,9 @@ int launch_mixed_score_attn(const void*, long, const void*, const void*,
                             void*, long, float*, long, float*, float*, float*,
                             int, int, int, int, int, int, int, int, int,
                             hipStream_t);
-int launch_group_topk_gate(const float*, float*, int*, long, int, int, int,
-                           int, int, int, hipStream_t);
+int launch_group_topk_gate(const float*, const float*, float*, int*, long,
+                           int, int, int, int, int, int, int, float,
+                           hipStream_t);
 int launch_attn_prefill_paged_mixed(
     const unsigned short*, long, const unsigned short*, const unsigned short*,
     const int*, const int*, const int*, unsigned short*, long, int, int, int,
@@ -425,7 +426,9 @@ void mixed_score_attn(const Tensor& q, const Tensor& k_cache,
 
 std::vector<Tensor> group_topk_gate(const Tensor& logits, int64_t top_k,
                                     int64_t n_groups, int64_t keep,
-                                    bool sigmoid, int64_t group_top) {
+                                    bool sigmoid, int64_t group_top,
+                                    const std::optional<Tensor>& choice_bias,
+                                    bool renorm, double route_scale) {
     check_f32(logits, "logits");
     TORCH_CHECK(logits.dim() == 2);
     const long T = logits.size(0);
@@ -435,13 +438,21 @@ std::vector<Tensor> group_topk_gate(const Tensor& logits, int64_t top_k,
                 top_k <= keep * (E / n_groups),
                 "experts must split into equal groups and the kept groups "
                 "must hold top_k experts");
+    TORCH_CHECK(n_groups == 1 || n_groups <= 64, "at most 64 groups");
+    const float* cb = nullptr;
+    if (choice_bias.has_value()) {
+        check_f32(*choice_bias, "choice_bias");
+        TORCH_CHECK(choice_bias->numel() == E);
+        cb = choice_bias->data_ptr<float>();
+    }
     Tensor w = torch::empty({T, top_k}, logits.options());
     Tensor idx = torch::empty({T, top_k},
                               logits.options().dtype(torch::kInt32));
     const int rc = launch_group_topk_gate(
-        logits.data_ptr<float>(), w.data_ptr<float>(), idx.data_ptr<int>(), T,
-        E, (int)top_k, (int)n_groups, (int)keep, (int)group_top,
-        sigmoid ? 1 : 0, stream());
+        logits.data_ptr<float>(), cb, w.data_ptr<float>(),
+        idx.data_ptr<int>(), T, E, (int)top_k, (int)n_groups, (int)keep,
+        (int)group_top, sigmoid ? 1 : 0, renorm ? 1 : 0, (float)route_scale,
+        stream());
     TORCH_CHECK(rc == 0, "group_topk_gate: too many experts for one "
                          "workgroup's LDS");
     return {w, idx};

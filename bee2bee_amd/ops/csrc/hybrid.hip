@@ -265,9 +265,10 @@ __global__ void canon_state_kernel(const T* __restrict__ h, long hs,
 
 // ----------------------------------------------------- latent cache store
 // Per token: cache row = [unit(kv[:C]) * w | rotate(kv[C:])]; q's rotated
-// parts are rotated in place. Rotation pairs dim i with i + dims/2 over the
-// first `dims` coords of the R-wide part; the rest pass through.
-template <typename T>
+// parts are rotated in place. Rotation pairs dim i with i + dims/2 (INTER:
+// 2i with 2i + 1) over the first `dims` coords of the R-wide part; the rest
+// pass through.
+template <typename T, bool INTER>
 __global__ void latent_rope_store_kernel(
     T* __restrict__ q_rot, long q_tok_stride, long q_head_stride, int H,
     const T* __restrict__ kv, long kv_stride, const float* __restrict__ w,
@@ -292,12 +293,14 @@ __global__ void latent_rope_store_kernel(
     const float* cs = cos_t + (long)p * half;
     const float* sn = sin_t + (long)p * half;
     for (int i = threadIdx.x; i < R; i += blockDim.x) {
+        // pair j, its other coordinate ip, and whether i is the first of it
+        const bool first = INTER ? (i & 1) == 0 : i < half;
+        const int j = INTER ? i >> 1 : (first ? i : i - half);
+        const int ip = INTER ? i ^ 1 : (first ? i + half : i - half);
         float o;
-        if (i < half) {
-            o = ldf(row + C + i) * cs[i] - ldf(row + C + i + half) * sn[i];
-        } else if (i < dims) {
-            const int j = i - half;
-            o = ldf(row + C + i) * cs[j] + ldf(row + C + j) * sn[j];
+        if (i < dims) {
+            const float b = ldf(row + C + ip) * sn[j];
+            o = ldf(row + C + i) * cs[j] + (first ? -b : b);
         } else {
             o = ldf(row + C + i);
         }
@@ -308,9 +311,10 @@ __global__ void latent_rope_store_kernel(
     for (int i = threadIdx.x; i < H * half; i += blockDim.x) {
         const int hh = i / half, j = i - hh * half;
         T* qh = qt + hh * q_head_stride;
-        const float u = ldf(qh + j), v = ldf(qh + j + half);
-        stf(qh + j, u * cs[j] - v * sn[j]);
-        stf(qh + j + half, v * cs[j] + u * sn[j]);
+        const int ia = INTER ? 2 * j : j, ib = INTER ? 2 * j + 1 : j + half;
+        const float u = ldf(qh + ia), v = ldf(qh + ib);
+        stf(qh + ia, u * cs[j] - v * sn[j]);
+        stf(qh + ib, v * cs[j] + u * sn[j]);
     }
 }
 
@@ -779,17 +783,16 @@ extern "C" void launch_latent_rope_store(
     void* q_rot, long q_tok_stride, long q_head_stride, int H, const void* kv,
     long kv_stride, const float* w, int C, int R, int dims, float eps,
     const int* positions, const float* cos_t, const float* sin_t, void* cache,
-    const int* slot_mapping, long T, int f32, hipStream_t s) {
+    const int* slot_mapping, int inter, long T, int f32, hipStream_t s) {
     if (T == 0) return;
     const int th = 256;
-    if (f32)
-        latent_rope_store_kernel<float><<<T, th, 0, s>>>(
-            (float*)q_rot, q_tok_stride, q_head_stride, H, (const float*)kv,
-            kv_stride, w, C, R, dims, eps, positions, cos_t, sin_t,
-            (float*)cache, slot_mapping);
-    else
-        latent_rope_store_kernel<unsigned short><<<T, th, 0, s>>>(
-            (unsigned short*)q_rot, q_tok_stride, q_head_stride, H,
-            (const unsigned short*)kv, kv_stride, w, C, R, dims, eps,
-            positions, cos_t, sin_t, (unsigned short*)cache, slot_mapping);
+#define LRS_LAUNCH(TT, I)                                                     \
+    latent_rope_store_kernel<TT, I><<<T, th, 0, s>>>(                         \
+        (TT*)q_rot, q_tok_stride, q_head_stride, H, (const TT*)kv, kv_stride, \
+        w, C, R, dims, eps, positions, cos_t, sin_t, (TT*)cache, slot_mapping)
+    if (f32 && inter) LRS_LAUNCH(float, true);
+    else if (f32) LRS_LAUNCH(float, false);
+    else if (inter) LRS_LAUNCH(unsigned short, true);
+    else LRS_LAUNCH(unsigned short, false);
+#undef LRS_LAUNCH
 }

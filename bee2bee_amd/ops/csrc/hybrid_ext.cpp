@@ -29,7 +29,7 @@ void launch_canon_conv(const void*, const float*, void*, const int*,
 void launch_latent_rope_store(void*, long, long, int, const void*, long,
                               const float*, int, int, int, float, const int*,
                               const float*, const float*, void*, const int*,
-                              long, int, hipStream_t);
+                              int, long, int, hipStream_t);
 int launch_latent_attn(const void*, const void*, long, long, const void*,
                        long, const void*, const int*, int, const int*,
                        const int*, void*, float*, float*, int, int, int, int,
@@ -72,11 +72,13 @@ int launch_attn_prefill_paged_sink(const unsigned short*, long,
                                    const int*, const int*, unsigned short*,
                                    long, int, int, int, int, int, int, int,
                                    const float*, float, int,
-                                   const unsigned short*, long, hipStream_t);
+                                   const unsigned short*, long, const float*,
+                                   hipStream_t);
 int launch_sink_attn(const void*, long, const void*, const void*, const int*,
                      int, const int*, const int*, const float*, void*, long,
                      float, float*, float*, int, int, int, int, int, int, int,
-                     int, int, const void*, long, hipStream_t);
+                     int, int, const void*, long, const float*,
+                     hipStream_t);
 }
 
 namespace {
@@ -217,7 +219,7 @@ void latent_rope_store(Tensor& q_rot, const Tensor& kv, const Tensor& kv_norm,
                        double eps, int64_t kv_rank, int64_t rope_dims,
                        const Tensor& positions, const Tensor& cos_t,
                        const Tensor& sin_t, Tensor& cache,
-                       const Tensor& slot_mapping) {
+                       const Tensor& slot_mapping, bool interleaved) {
     const int c = act_code(kv, "kv");
     check_f32(kv_norm, "kv_norm");
     check_f32(cos_t, "cos");
@@ -244,11 +246,11 @@ void latent_rope_store(Tensor& q_rot, const Tensor& kv, const Tensor& kv_norm,
         kv_norm.data_ptr<float>(), C, R, (int)rope_dims, (float)eps,
         positions.data_ptr<int>(), cos_t.data_ptr<float>(),
         sin_t.data_ptr<float>(), cache.data_ptr(),
-        slot_mapping.data_ptr<int>(), T, c, stream());
+        slot_mapping.data_ptr<int>(), interleaved ? 1 : 0, T, c, stream());
 }
 
 Tensor latent_attn(const Tensor& q_abs, const Tensor& q_rot,
-                   const Tensor& gate, const Tensor& cache,
+                   const std::optional<Tensor>& gate, const Tensor& cache,
                    const Tensor& block_table, const Tensor& positions,
                    const Tensor& seq_idx, const Tensor& cu, int64_t window,
                    double scale, int64_t max_qlen,
@@ -265,9 +267,16 @@ Tensor latent_attn(const Tensor& q_abs, const Tensor& q_rot,
                 q_rot.dim() == 3 && q_rot.size(0) == Tn &&
                 q_rot.size(1) == H && q_rot.stride(2) == 1);
     const int R = (int)q_rot.size(2);
-    TORCH_CHECK(gate.is_cuda() && gate.scalar_type() == q_abs.scalar_type() &&
-                gate.dim() == 2 && gate.size(0) == Tn && gate.size(1) == H &&
-                gate.stride(1) == 1);
+    const void* gp = nullptr;
+    long gate_tok = 0;
+    if (gate.has_value()) {
+        TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 &&
+                    gate->scalar_type() == q_abs.scalar_type() &&
+                    gate->size(0) == Tn && gate->size(1) == H &&
+                    gate->stride(1) == 1);
+        gp = gate->data_ptr();
+        gate_tok = gate->stride(0);
+    }
     TORCH_CHECK(cache.is_cuda() && cache.scalar_type() == q_abs.scalar_type() &&
                 cache.is_contiguous() && cache.dim() == 3 &&
                 cache.size(2) == C + R);
@@ -308,7 +317,7 @@ Tensor latent_attn(const Tensor& q_abs, const Tensor& q_rot,
         }
         const int rc = launch_latent_attn_mfma(
             q_abs.data_ptr(), q_rot.data_ptr(), q_rot.stride(0),
-            q_rot.stride(1), gate.data_ptr(), gate.stride(0),
+            q_rot.stride(1), gp, gate_tok,
             cache.data_ptr(), block_table.data_ptr<int>(),
             (int)block_table.size(1), cu.data_ptr<int>(),
             positions.data_ptr<int>(), seq_idx.data_ptr<int>(),
@@ -327,7 +336,7 @@ Tensor latent_attn(const Tensor& q_abs, const Tensor& q_rot,
     if (splits > 1) alloc_parts(splits);
     const int rc = launch_latent_attn(
         q_abs.data_ptr(), q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1),
-        gate.data_ptr(), gate.stride(0), cache.data_ptr(),
+        gp, gate_tok, cache.data_ptr(),
         block_table.data_ptr<int>(), (int)block_table.size(1),
         positions.data_ptr<int>(), seq_idx.data_ptr<int>(), out.data_ptr(),
         pa, pm, (int)splits, Tn, H, C, R, (int)cache.size(1), (int)window,
@@ -655,7 +664,8 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
                const Tensor& seq_idx, const Tensor& cu,
                const std::optional<Tensor>& sink, int64_t window, Tensor& out,
                double out_scale, int64_t max_qlen,
-               const std::optional<Tensor>& head_gate) {
+               const std::optional<Tensor>& head_gate,
+               const std::optional<Tensor>& dist) {
     const int c = act_code(q, "q");
     check_i32(block_table, "block_table");
     check_i32(positions, "positions");
@@ -690,6 +700,13 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
         hg = head_gate->data_ptr();
         hg_tok = head_gate->stride(0);
     }
+    const float* dp = nullptr;
+    if (dist.has_value()) {
+        check_f32(*dist, "dist");
+        TORCH_CHECK(dist->dim() == 2 && dist->size(0) == 2 &&
+                    dist->size(1) == H);
+        dp = dist->data_ptr<float>();
+    }
     // bf16 prompt portions with head size 64/128 run on the matrix cores
     // (the dense models' paged prefill kernel, with the weights as a bf16
     // pair, window-aware tile skipping, and the sink and head gate in its
@@ -710,7 +727,7 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
             (unsigned short*)out.data_ptr(), out.stride(0), (int)B, H, G, D,
             (int)block_table.size(1), bs, (int)max_qlen, sk,
             (float)out_scale, (int)window, (const unsigned short*)hg, hg_tok,
-            stream());
+            dp, stream());
         TORCH_CHECK(rc == 0, "sink_attn: matrix-core path refused a shape "
                              "its guard admitted");
         return;
@@ -738,7 +755,7 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
         block_table.data_ptr<int>(), (int)block_table.size(1),
         positions.data_ptr<int>(), seq_idx.data_ptr<int>(), sk,
         out.data_ptr(), out.stride(0), (float)out_scale, pa, pm, (int)splits,
-        Tn, H, G, D, Dv, bs, (int)window, c, hg, hg_tok, stream());
+        Tn, H, G, D, Dv, bs, (int)window, c, hg, hg_tok, dp, stream());
     TORCH_CHECK(rc == 0, "sink_attn: head sizes must be <= 256");
 }
 
@@ -786,5 +803,6 @@ void register_hybrid_ops(pybind11::module_& m) {
           pybind11::arg("cu_seqlens"), pybind11::arg("sink"),
           pybind11::arg("window"), pybind11::arg("out"),
           pybind11::arg("out_scale"), pybind11::arg("max_qlen"),
-          pybind11::arg("head_gate") = std::nullopt);
+          pybind11::arg("head_gate") = std::nullopt,
+          pybind11::arg("dist") = std::nullopt);
 }

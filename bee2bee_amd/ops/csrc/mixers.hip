@@ -138,7 +138,8 @@ latent_attn_kernel(const T* __restrict__ q_abs,   // [H, Tn, C]
         }
         return;
     }
-    const float g = 1.f / (1.f + expf(-ldf(gate + (long)t * gate_tok + h)));
+    const float g =
+        gate ? 1.f / (1.f + expf(-ldf(gate + (long)t * gate_tok + h))) : 1.f;
     float r = g / l;
     if (sink) {
         // a logit that joins the denominator without key or value
@@ -372,8 +373,8 @@ latent_attn_mfma_kernel(const unsigned short* __restrict__ q_abs,
                     part_ml[row * 2 + 1] = l_run[r];
                 }
             } else {
-                const float g = 1.f / (1.f + expf(-bf2f(
-                    gate[(long)s0 * gate_tok + hh])));
+                const float g = gate ? 1.f / (1.f + expf(-bf2f(
+                    gate[(long)s0 * gate_tok + hh]))) : 1.f;
                 float inv = l_run[r] > 0.f ? g / l_run[r] : 0.f;
                 if (sink) {
                     const float sk = sink[hh];
@@ -396,8 +397,8 @@ latent_attn_mfma_kernel(const unsigned short* __restrict__ q_abs,
     for (int r = 0; r < 4; ++r) {
         const int qrow = q0 + lg * 4 + r;
         if (qrow >= QL) continue;
-        const float g = 1.f / (1.f + expf(-bf2f(
-            gate[(long)(s0 + qrow) * gate_tok + h])));
+        const float g = gate ? 1.f / (1.f + expf(-bf2f(
+            gate[(long)(s0 + qrow) * gate_tok + h]))) : 1.f;
         float inv = l_run[r] > 0.f ? g / l_run[r] : 0.f;
         if (sink) {
             const float sk = sink[h];
@@ -440,7 +441,8 @@ latent_attn_combine_kernel(const float* __restrict__ part_acc,
     const float w = l > 0.f ? expf(m - M) : 0.f;
     float L = wave_sum(l * w);
     if (sink) L += expf(sink[h] - M);
-    const float g = 1.f / (1.f + expf(-ldf(gate + (long)t * gate_tok + h)));
+    const float g =
+        gate ? 1.f / (1.f + expf(-ldf(gate + (long)t * gate_tok + h))) : 1.f;
     const float r = g / L;
     T* o = out + ((long)h * Tn + t) * C;
     // uniform trip count: every lane takes part in every shuffle
@@ -1012,7 +1014,8 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
                  long out_tok, float out_scale, float* __restrict__ part_acc,
                  float* __restrict__ part_ml, int Tn, int H, int G, int D,
                  int Dv, int bs, int window,
-                 const T* __restrict__ head_gate, long hg_tok) {
+                 const T* __restrict__ head_gate, long hg_tok,
+                 const float* __restrict__ dist) {
     extern __shared__ __attribute__((aligned(16))) float sa_q[];
     const int wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     const int t = blockIdx.x;
@@ -1033,11 +1036,13 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
         qv[i] = ldf(q + (long)t * q_tok + (long)h0 * D + i);
     WAVE_LDS_SYNC();
     const int* bt = block_table + (long)seq_idx[t] * bt_stride;
-    float m[REP], l[REP], acc[REP][DPL];
+    float m[REP], l[REP], acc[REP][DPL], da[REP], db[REP];
 #pragma unroll
     for (int r = 0; r < REP; ++r) {
         m[r] = -INFINITY;
         l[r] = 0.f;
+        da[r] = dist ? dist[h0 + r] : 0.f;
+        db[r] = dist ? dist[H + h0 + r] : 0.f;
 #pragma unroll
         for (int i = 0; i < DPL; ++i) acc[r][i] = 0.f;
     }
@@ -1053,6 +1058,12 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
         for (int r = 0; r < REP; ++r) sc[r] = 0.f;
         const int nk = min(WAVE, khi - j0);
         if (valid) SaDots<T, REP>::run(k_cache + (long)row * D, qv, D, sc);
+        if (dist) {
+            const float d = (float)(p - jc);
+#pragma unroll
+            for (int r = 0; r < REP; ++r)
+                sc[r] -= da[r] * logf(1.f + db[r] * d);
+        }
 #pragma unroll
         for (int r = 0; r < REP; ++r) {
             const float s = valid ? sc[r] : -INFINITY;
@@ -1407,7 +1418,7 @@ extern "C" int launch_delta_rule(const float* q, const float* k, long qk_tok,
         (const TT*)q, q_tok, (const TT*)k_cache, (const TT*)v_cache,          \
         block_table, bt_stride, positions, seq_idx, sink, (TT*)out, out_tok,  \
         out_scale, part_acc, part_ml, Tn, H, G, D, Dv, bs, window,            \
-        (const TT*)head_gate, hg_tok)
+        (const TT*)head_gate, hg_tok, dist)
 
 #define SA_CASE(N, P)                                                         \
     if (dpl == N && pair == P) {                                              \
@@ -1426,7 +1437,7 @@ static int sink_attn_dispatch(const void* q, long q_tok, const void* k_cache,
                               float* part_acc, float* part_ml, int splits,
                               int Tn, int H, int G, int D, int Dv, int bs,
                               int window, const void* head_gate, long hg_tok,
-                              hipStream_t s) {
+                              const float* dist, hipStream_t s) {
     // even value sizes: a lane owns coordinate pairs (one load for two)
     const bool pair = Dv % 2 == 0;
     int dpl = pair ? 2 * ((Dv + 2 * WAVE - 1) / (2 * WAVE))
@@ -1452,8 +1463,9 @@ static int sink_attn_dispatch(const void* q, long q_tok, const void* k_cache,
 }
 
 // head_gate (optional, activation type, [Tn, H] with row stride hg_tok):
-// head h's output times sigmoid(head_gate[t, h]). Returns nonzero when a
-// head size exceeds 256.
+// head h's output times sigmoid(head_gate[t, h]). dist (optional, fp32
+// [2, H] = (a, b)): a_h ln(1 + b_h d) is taken off a score whose key lies d
+// positions back. Returns nonzero when a head size exceeds 256.
 extern "C" int launch_sink_attn(const void* q, long q_tok,
                                 const void* k_cache, const void* v_cache,
                                 const int* block_table, int bt_stride,
@@ -1463,18 +1475,18 @@ extern "C" int launch_sink_attn(const void* q, long q_tok,
                                 float* part_ml, int splits, int Tn, int H,
                                 int G, int D, int Dv, int bs, int window,
                                 int f32, const void* head_gate, long hg_tok,
-                                hipStream_t s) {
+                                const float* dist, hipStream_t s) {
     if (D > SA_MAXD || Dv > SA_MAXD) return 1;
     if (Tn == 0) return 0;
     if (f32)
         return sink_attn_dispatch<float>(
             q, q_tok, k_cache, v_cache, block_table, bt_stride, positions,
             seq_idx, sink, out, out_tok, out_scale, part_acc, part_ml, splits,
-            Tn, H, G, D, Dv, bs, window, head_gate, hg_tok, s);
+            Tn, H, G, D, Dv, bs, window, head_gate, hg_tok, dist, s);
     return sink_attn_dispatch<unsigned short>(
         q, q_tok, k_cache, v_cache, block_table, bt_stride, positions,
         seq_idx, sink, out, out_tok, out_scale, part_acc, part_ml, splits, Tn,
-        H, G, D, Dv, bs, window, head_gate, hg_tok, s);
+        H, G, D, Dv, bs, window, head_gate, hg_tok, dist, s);
 }
 
 // ---------------------------------------------------------------------------

@@ -403,30 +403,34 @@ def latent_rope_store(q_rot: torch.Tensor, kv: torch.Tensor,
                       kv_norm: torch.Tensor, eps: float, kv_rank: int,
                       rope_dims: int, positions: torch.Tensor,
                       cos: torch.Tensor, sin: torch.Tensor,
-                      cache: torch.Tensor, slot_mapping: torch.Tensor) -> None:
+                      cache: torch.Tensor, slot_mapping: torch.Tensor,
+                      interleaved: bool = False) -> None:
     """q_rot [T, H, R] (view, rotated in place); kv [T, kv_rank + R] (view):
     cache row = [rmsnorm(kv[:kv_rank]) * kv_norm | rotate(kv[kv_rank:])].
-    cache [n_blocks, block_size, kv_rank + R]."""
+    cache [n_blocks, block_size, kv_rank + R]. Rotated pairs: (2i, 2i+1)
+    when interleaved, else (i, i + rope_dims/2)."""
     p = positions.long()
     c, s = cos[p], sin[p]                                   # [T, dims/2]
-    q_rot.copy_(_rot_half(q_rot.float(), c[:, None], s[:, None],
-                          rope_dims).to(q_rot.dtype))
+    rot = _rot_pairs if interleaved else _rot_half
+    q_rot.copy_(rot(q_rot.float(), c[:, None], s[:, None],
+                    rope_dims).to(q_rot.dtype))
     lat = kv[:, :kv_rank].float()
     lat = lat * torch.rsqrt(lat.pow(2).mean(-1, keepdim=True) + eps) * kv_norm
-    kr = _rot_half(kv[:, kv_rank:].float(), c, s, rope_dims)
+    kr = rot(kv[:, kv_rank:].float(), c, s, rope_dims)
     flat = cache.view(-1, cache.shape[-1])
     flat[slot_mapping.long()] = torch.cat([lat, kr], -1).to(cache.dtype)
 
 
-def latent_attn(q_abs: torch.Tensor, q_rot: torch.Tensor, gate: torch.Tensor,
-                cache: torch.Tensor, block_table: torch.Tensor,
+def latent_attn(q_abs: torch.Tensor, q_rot: torch.Tensor,
+                gate: Optional[torch.Tensor], cache: torch.Tensor, block_table: torch.Tensor,
                 positions: torch.Tensor, seq_idx: torch.Tensor,
                 cu_seqlens: torch.Tensor, window: int,
                 scale: float,
                 sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Windowed softmax attention in the latent space (one shared key/value
     row per token). q_abs [H, T, C] (queries already multiplied by the key
-    up-projection), q_rot [T, H, R], gate [T, H] raw (sigmoid applied here).
+    up-projection), q_rot [T, H, R], gate [T, H] raw (sigmoid applied here;
+    None: no gate).
     Row t at position p of sequence b sees cached positions
     max(0, p - window + 1) .. p (window 0: 0 .. p). sink fp32 [H]: exp(sink)
     joins the softmax denominator, unscaled, without a value. Returns
@@ -462,7 +466,9 @@ def latent_attn(q_abs: torch.Tensor, q_rot: torch.Tensor, gate: torch.Tensor,
             e = torch.exp(s - m)
             p = e / (e.sum(-1, keepdim=True) + torch.exp(sk - m))
         o = torch.einsum("hts,sc->htc", p, kv[:, :C])
-        out[:, lo:hi] = o * torch.sigmoid(gate[lo:hi].float()).t()[..., None]
+        if gate is not None:
+            o = o * torch.sigmoid(gate[lo:hi].float()).t()[..., None]
+        out[:, lo:hi] = o
     return out.to(q_abs.dtype)
 
 
@@ -994,22 +1000,27 @@ def silu_glu(gate_up: torch.Tensor) -> torch.Tensor:
 
 def group_topk_gate(logits: torch.Tensor, top_k: int, n_groups: int,
                     keep_groups: int, score: str = "softmax",
-                    group_top: int = 1) -> Tuple[torch.Tensor, torch.Tensor]:
+                    group_top: int = 1,
+                    choice_bias: Optional[torch.Tensor] = None,
+                    renorm: bool = False, route_scale: float = 1.0
+                    ) -> Tuple[torch.Tensor, torch.Tensor]:
     """Group-limited choice on expert scores. logits fp32 [T, E]: scores =
     softmax over all experts (score "softmax") or the sigmoid of each logit
     ("sigmoid"); experts form n_groups equal groups of neighbours, a group's
     score is the sum of its group_top largest expert scores, experts outside
     the best keep_groups groups cannot be chosen; the top_k remaining scores
     are the weights, as they are. -> (weights [T, k] fp32, idx [T, k] int32).
-    Fixed shapes and no host sync (graph-capturable)."""
+    choice_bias fp32 [E] joins the scores for the choice (groups included)
+    but not the weights; renorm: the weights are divided by their sum
+    (+ 1e-20); route_scale multiplies them last. Fixed shapes and no host sync (graph-capturable)."""
     T, E = logits.shape
     if score == "sigmoid":
         s = torch.sigmoid(logits.float())
     else:
         s = torch.softmax(logits.float(), dim=-1)
-    pick = s
+    pick = s if choice_bias is None else s + choice_bias.float()
     if n_groups > 1 and keep_groups < n_groups:
-        per = s.view(T, n_groups, E // n_groups)
+        per = pick.view(T, n_groups, E // n_groups)
         if group_top <= 1:
             gs = per.max(-1).values
         else:
@@ -1019,9 +1030,13 @@ def group_topk_gate(logits: torch.Tensor, top_k: int, n_groups: int,
         allow = torch.zeros(T, n_groups, dtype=torch.bool, device=s.device)
         allow.scatter_(1, top_g, True)
         allow = allow[:, :, None].expand(T, n_groups, E // n_groups)
-        pick = torch.where(allow.reshape(T, E), s, torch.full_like(s, -1.0))
+        pick = torch.where(allow.reshape(T, E), pick,
+                           torch.full_like(s, float("-inf")))
     idx = torch.topk(pick, top_k, dim=-1).indices
-    return s.gather(1, idx), idx.to(torch.int32)
+    w = s.gather(1, idx)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return w * route_scale, idx.to(torch.int32)
 
 
 # ------------------------------------------- gated parallel-form stacks
@@ -1107,9 +1122,11 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
              softcap: float, talk: Optional[torch.Tensor],
              sink: Optional[torch.Tensor],
              head_gate: Optional[torch.Tensor], window: int,
-             out: torch.Tensor) -> None:
+             out: torch.Tensor,
+             dist: Optional[torch.Tensor] = None) -> None:
     """Grouped-query attention over the pages. Scores q . k (the score
-    scale is already in q); softcap > 0: s <- softcap tanh(s / softcap);
+    scale is already in q); dist fp32 [2, H] = (a, b): s_h <- s_h -
+    a_h ln(1 + b_h d), d the distance between row and key; softcap > 0: s <- softcap tanh(s / softcap);
     talk fp32 [H, H]: s_h <- sum_g talk[h, g] s_g at every (row, key),
     BEFORE the softmax. Row t at position p of chunk b sees cached positions
     j <= p (j > p - window when window > 0). sink fp32 [H]: exp(sink_h)
@@ -1134,11 +1151,14 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         vals = v_cache[blk, :, kpos % bs].float()          # [S, G, Dv]
         qb = q[lo:hi].float().view(hi - lo, G, rep, D)
         s = torch.einsum("tgrd,sgd->grts", qb, keys).reshape(H, hi - lo, -1)
+        d = pos[:, None] - kpos[None, :]
+        if dist is not None:
+            a, r = dist.float()[:, :, None, None]
+            s = s - a * torch.log1p(r * d.clamp(min=0)[None])
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
         if talk is not None:
             s = torch.einsum("hg,gts->hts", talk.float(), s)
-        d = pos[:, None] - kpos[None, :]
         dead = d < 0
         if window > 0:
             dead = dead | (d >= window)
@@ -1233,3 +1253,67 @@ def gated_add_rmsnorm(resid: torch.Tensor, y1: torch.Tensor,
 def gelu_erf(x: torch.Tensor) -> torch.Tensor:
     """Exact gelu, x/2 (1 + erf(x / sqrt 2)), evaluated in fp32."""
     return torch.nn.functional.gelu(x.float()).to(x.dtype)
+
+
+# --------------------------------------------------- dynamic-tanh stacks
+#
+# Mechanisms of stacks whose sublayers are x += n_b(f(n_a(x))) with
+# n(x) = tanh(alpha x) * w + b: the norm pair around the fp32 residual
+# update, query/key norms over the whole projection with the page store, and
+# the expert activation of a step whose tokens run through every expert's
+# columns of one product.
+
+
+def tanh_norm(x: torch.Tensor, n, out_dtype: torch.dtype) -> torch.Tensor:
+    """n = (alpha, w, b): tanh(alpha x) * w + b, fp32 inside."""
+    a, w, b = n
+    return (torch.tanh(x.float() * a) * w + b).to(out_dtype)
+
+
+def add_tanh_norm(resid: torch.Tensor, y: Optional[torch.Tensor], post, pre,
+                  out_dtype: torch.dtype) -> Optional[torch.Tensor]:
+    """resid (fp32, in place) += tanh_norm(y, post) when y is given; returns
+    tanh_norm(resid, pre) (None if pre is)."""
+    if y is not None:
+        resid.add_(tanh_norm(y, post, torch.float32))
+    return None if pre is None else tanh_norm(resid, pre, out_dtype)
+
+
+def proj_norm_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
+                    q_norm: torch.Tensor, k_norm: torch.Tensor, v_unit: bool,
+                    eps: float, q_mult: float, k_cache: torch.Tensor,
+                    v_cache: torch.Tensor,
+                    slot_mapping: torch.Tensor) -> None:
+    """q [T, H, D] (view, rewritten in place): unit over ALL H * D numbers,
+    times q_norm [H * D] * q_mult. k [T, G, D] (view): unit over all G * D,
+    times k_norm, to k_cache [n_blocks, G, block, D]. v [T, G, Dv] (view) to
+    v_cache [n_blocks, G, block, Dv], each head first divided by its root
+    mean square when v_unit. unit = x / sqrt(mean(x^2) + eps)."""
+    T, H, D = q.shape
+    G, bs = k.shape[1], k_cache.shape[2]
+
+    def un(x):
+        return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+    qn = un(q.float().reshape(T, H * D)) * q_norm * q_mult
+    kn = un(k.float().reshape(T, G * D)) * k_norm
+    q.copy_(qn.view(T, H, D).to(q.dtype))
+    vn = un(v.float()) if v_unit else v
+    slot = slot_mapping.long()
+    blk, off = slot // bs, slot % bs
+    k_cache[blk, :, off] = kn.view(T, G, D).to(k_cache.dtype)
+    v_cache[blk, :, off] = vn.to(v_cache.dtype)
+
+
+def routed_silu_glu(gu: torch.Tensor, weights: torch.Tensor,
+                    idx: torch.Tensor) -> torch.Tensor:
+    """gu [T, E, 2I] (gate | up of every expert) -> [T, E * I]: silu(gate) *
+    up * the token's weight for that expert, zero where idx [T, k] does not
+    name it."""
+    T, E, I2 = gu.shape
+    g, u = gu.float().chunk(2, dim=-1)
+    full = torch.zeros(T, E, dtype=torch.float32, device=gu.device)
+    full.scatter_(1, idx.long(), weights)
+    y = torch.nn.functional.silu(g) * u * full[..., None]
+    y = torch.where((full != 0)[..., None], y, torch.zeros_like(y))
+    return y.to(gu.dtype).view(T, E * (I2 // 2))
