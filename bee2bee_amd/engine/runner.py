@@ -286,53 +286,60 @@ class Runner:
             and H % 128 == 0 and I % 128 == 0
             and T <= self.MOE_GROUPED_ROWS * E // top_k
         )
-        # the padded bmm is CPU-only: the library's batched TN bf16 product
-        # is not usable on gfx950 at these sizes — GPU sizes above the
-        # grouped range take the per-expert GEMM loop below, whose plain TN
-        # GEMMs are solid
+        # the padded bmm is CPU-only: GPU sizes above the grouped range take
+        # plain per-expert GEMMs on sorted rows
         use_bmm = x.device.type != "cuda"
-        if T <= self.MOE_BMM_MAX_TOKENS and (use_grouped or use_bmm):
-            # counting sort from one-hot cumsums: every op here (one_hot,
-            # cumsum, gather, index_copy) is hipGraph-capture-safe —
-            # torch.bincount/argsort are not
+        if use_grouped:
+            # grouped-GEMM HIP kernel (default in this range): segment sizes
+            # stay on the device, no host sync, static shapes -> the whole
+            # MoE decode step hipGraph-captures; measured 3.8 TB/s of W per
+            # projection
+            pos, tok, offs = ops.moe_sort(idx, E)
+            gu = ops.grouped_gemm(x.index_select(0, tok), lw.moe_w_gate_up,
+                                  offs)
+            y = ops.grouped_gemm(act_fn(gu), lw.moe_w_down, offs)
+            return ops.moe_combine(y, pos, weights)
+        if T <= self.MOE_BMM_MAX_TOKENS and use_bmm:
+            # padded per-expert bmm: weights read once per expert, flops
+            # proportional to max routed count. M aligns up to 16 (<2%
+            # padded flops)
             k = top_k
             S = T * k
             flat_e = idx.reshape(-1).to(torch.int64)  # slot s -> expert
             oh = F.one_hot(flat_e, E)  # [S, E]
             counts = oh.sum(0)
-            offs_excl = counts.cumsum(0) - counts
             rank = (oh.cumsum(0) - oh).gather(1, flat_e.unsqueeze(1)).squeeze(1)
-            pos = (offs_excl[flat_e] + rank).to(torch.int64)  # dest row
             tok = torch.arange(S, device=x.device, dtype=torch.int64) // k
-            if use_grouped:
-                # grouped-GEMM HIP kernel (default in this range): no host
-                # sync, static shapes -> the whole MoE decode step hipGraph-
-                # captures; measured 3.8 TB/s of W per projection
-                offsets = torch.zeros(E + 1, dtype=torch.int32, device=x.device)
-                offsets[1:] = counts.cumsum(0).to(torch.int32)
-                x_sorted = torch.empty(S, H, dtype=x.dtype, device=x.device)
-                x_sorted.index_copy_(0, pos, x[tok])
-                gu = ops.grouped_gemm(x_sorted, lw.moe_w_gate_up, offsets)
-                act = act_fn(gu)
-                y = ops.grouped_gemm(act, lw.moe_w_down, offsets)  # [S, H]
-                contrib = y[pos].float()  # back to slot order
-            else:
-                # padded per-expert bmm: weights read once per expert, flops
-                # proportional to max routed count; counts.max() is one host
-                # sync per MoE layer (so no hipGraph above the dense range).
-                # M aligns up to 16 (<2% padded flops)
-                C = (int(counts.max()) + 15) & ~15
-                padded = torch.zeros(E, C, H, dtype=x.dtype, device=x.device)
-                padded[flat_e, rank] = x[tok]
-                gu = torch.bmm(padded, lw.moe_w_gate_up.transpose(1, 2))
-                act = act_fn(gu.reshape(E * C, U)).view(E, C, I)
-                y = torch.bmm(act, lw.moe_w_down.transpose(1, 2))  # [E,C,H]
-                contrib = y[flat_e, rank].float()  # [S, H] slot order
+            C = (int(counts.max()) + 15) & ~15
+            padded = torch.zeros(E, C, H, dtype=x.dtype, device=x.device)
+            padded[flat_e, rank] = x[tok]
+            gu = torch.bmm(padded, lw.moe_w_gate_up.transpose(1, 2))
+            act = act_fn(gu.reshape(E * C, U)).view(E, C, I)
+            y = torch.bmm(act, lw.moe_w_down.transpose(1, 2))  # [E,C,H]
+            contrib = y[flat_e, rank].float()  # [S, H] slot order
             out = torch.zeros(T, H, dtype=torch.float32, device=x.device)
             out.index_add_(
                 0, tok, contrib * weights.reshape(-1).unsqueeze(-1)
             )
             return out.to(x.dtype)
+
+        if x.device.type == "cuda":
+            # pairs sorted by expert on the device, one host read of the
+            # segment bounds, one plain GEMM per expert and projection on
+            # neighbouring rows, one activation, one weighted sum
+            pos, tok, offs = ops.moe_sort(idx, E)
+            x_sorted = x.index_select(0, tok)
+            bounds = offs.tolist()
+            gu = torch.empty(T * top_k, U, dtype=x.dtype, device=x.device)
+            y = torch.empty(T * top_k, H, dtype=x.dtype, device=x.device)
+            segs = [(e, a, b) for e, (a, b) in
+                    enumerate(zip(bounds, bounds[1:])) if b > a]
+            for e, a, b in segs:
+                torch.mm(x_sorted[a:b], lw.moe_w_gate_up[e].t(), out=gu[a:b])
+            act = act_fn(gu)
+            for e, a, b in segs:
+                torch.mm(act[a:b], lw.moe_w_down[e].t(), out=y[a:b])
+            return ops.moe_combine(y, pos, weights)
 
         out = torch.zeros_like(x, dtype=torch.float32)
         for e in range(E):

@@ -617,7 +617,26 @@ def proj_norm_store(q, k, v, q_norm, k_norm, v_unit: bool, eps: float,
                               k_cache, v_cache, slot_mapping)
 
 
+
+# ------------------------------------------------------- routed experts
+
+
 def routed_silu_glu(gu, weights, idx):
     if _use_hip(gu):
         return require_hip().routed_silu_glu(gu, weights, idx)
     return reference.routed_silu_glu(gu, weights, idx)
+
+
+def moe_sort(idx, n_experts: int):
+    """(token, choice) pairs in expert order: -> pos [T, k] (row of each
+    pair), tok [T * k] (token of each row), offs [E + 1], int32."""
+    if _use_hip(idx):
+        return tuple(require_hip().moe_sort(idx, n_experts))
+    return reference.moe_sort(idx, n_experts)
+
+
+def moe_combine(y, pos, weights):
+    """out[t] = sum_j weights[t, j] * y[pos[t, j]], summed in fp32."""
+    if _use_hip(y):
+        return require_hip().moe_combine(y, pos, weights)
+    return reference.moe_combine(y, pos, weights)

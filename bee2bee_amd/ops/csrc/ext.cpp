@@ -52,7 +52,7 @@ void launch_mfma_probe_fp8(const unsigned char*, const unsigned char*,
                            float*, hipStream_t);
 void launch_grouped_gemm(const unsigned short*, const unsigned short*,
                          const int*, unsigned short*, int, int, int, int,
-                         hipStream_t);
+                         long, long, hipStream_t);
 void launch_bw_linear(const unsigned short*, long, float*, hipStream_t);
 void launch_bw_rowperlane(const unsigned short*, long, int, int, float*,
                           hipStream_t);
@@ -331,7 +331,10 @@ Tensor grouped_gemm(const Tensor& x, const Tensor& w, const Tensor& offs) {
     check_bf16(x, "x");
     check_bf16(w, "w");
     TORCH_CHECK(offs.scalar_type() == torch::kInt32 && offs.is_contiguous());
-    TORCH_CHECK(x.is_contiguous() && w.is_contiguous());
+    // w may be a view: unit stride along K, 16-byte aligned rows
+    TORCH_CHECK(x.is_contiguous() && w.dim() == 3 && w.stride(2) == 1 &&
+                w.stride(1) % 8 == 0 && w.stride(0) % 8 == 0 &&
+                reinterpret_cast<uintptr_t>(w.data_ptr()) % 16 == 0);
     const int S = x.size(0), K = x.size(1);
     const int E = w.size(0), N = w.size(1);
     TORCH_CHECK(w.size(2) == K, "K mismatch");
@@ -341,7 +344,8 @@ Tensor grouped_gemm(const Tensor& x, const Tensor& w, const Tensor& offs) {
     Tensor out = torch::empty({S, N}, x.options());
     if (S > 0)
         launch_grouped_gemm(bf16p(x), bf16p(w), offs.data_ptr<int>(),
-                            bf16p_mut(out), E, S, N, K, stream());
+                            bf16p_mut(out), E, S, N, K, w.stride(0),
+                            w.stride(1), stream());
     return out;
 }
 
@@ -399,12 +403,14 @@ void register_hybrid_ops(pybind11::module_& m);  // hybrid_ext.cpp
 void register_sandwich_ops(pybind11::module_& m);  // sandwich_ext.cpp
 void register_gated_ops(pybind11::module_& m);  // gated_ext.cpp
 void register_tanh_ops(pybind11::module_& m);  // tanh_ext.cpp
+void register_moe_ops(pybind11::module_& m);  // moe_ext.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     register_hybrid_ops(m);
     register_sandwich_ops(m);
     register_gated_ops(m);
     register_tanh_ops(m);
+    register_moe_ops(m);
     m.def("rmsnorm", &rmsnorm, "fused RMSNorm (bf16)");
     m.def("fused_add_rmsnorm", &fused_add_rmsnorm,
           "residual += x; y = rmsnorm(residual)");

@@ -419,10 +419,10 @@ group_topk_gate_kernel(const float* __restrict__ logits,
     float* gsc = gt_s + (long)E * GT_THREADS + threadIdx.x;  // [n_groups]
     const int st = GT_THREADS;
     const float* z = logits + t * E;
+    float m = -INFINITY, sum = 0.f;        // softmax form
     if (sigmoid) {
         for (int e = 0; e < E; ++e) sc[e * st] = sigmoid_f(z[e]);
     } else {
-        float m = -INFINITY, sum = 0.f;
         for (int e = 0; e < E; ++e) m = fmaxf(m, z[e]);
         for (int e = 0; e < E; ++e) {
             const float x = expf(z[e] - m);
@@ -482,8 +482,8 @@ group_topk_gate_kernel(const float* __restrict__ logits,
         }
         if (be < 0) be = 0;                // only when scores are not numbers
         float w = best;
-        if (choice_bias) w = sigmoid ? sigmoid_f(z[be])
-                                     : best - choice_bias[be];
+        if (choice_bias)
+            w = sigmoid ? sigmoid_f(z[be]) : expf(z[be] - m) / sum;
         w_out[t * top_k + it] = w;
         idx_out[t * top_k + it] = be;
         total += w;

@@ -48,10 +48,10 @@
 
 __global__ __launch_bounds__(GG_BLOCK) void grouped_gemm_kernel(
     const unsigned short* __restrict__ x,   // [S, K]
-    const unsigned short* __restrict__ w,   // [E, N, K]
+    const unsigned short* __restrict__ w,   // [E, N, K], strides we, wn, 1
     const int* __restrict__ offs,           // [E+1]
     unsigned short* __restrict__ out,       // [S, N]
-    int N, int K) {
+    int N, int K, long we, long wn) {
     const int e = blockIdx.y;
     const int n0 = blockIdx.x * GG_BN;
     const int m_lo = offs[e];
@@ -80,7 +80,7 @@ __global__ __launch_bounds__(GG_BLOCK) void grouped_gemm_kernel(
     // conflict-free)
     const int ws_col = tid >> 3;
     const int ws_d = (tid & 7) * 8;
-    const unsigned short* wrow = w + ((long)e * N + n0 + ws_col) * K + ws_d;
+    const unsigned short* wrow = w + e * we + (n0 + ws_col) * wn + ws_d;
     const int ng = K / GG_KG;   // K % 128 == 0 checked host-side
 
     for (int pass = m_lo; pass < m_hi; pass += GG_MROWS) {
@@ -178,9 +178,10 @@ __global__ __launch_bounds__(GG_BLOCK) void grouped_gemm_kernel(
 
 extern "C" void launch_grouped_gemm(
     const unsigned short* x, const unsigned short* w, const int* offs,
-    unsigned short* out, int E, int S, int N, int K, hipStream_t stream) {
+    unsigned short* out, int E, int S, int N, int K, long we, long wn,
+    hipStream_t stream) {
     dim3 grid(N / GG_BN, E);
     const int smem = 2 * (GG_MROWS + GG_BN) * (GG_KG + GG_PAD) * 2;
     hipLaunchKernelGGL(grouped_gemm_kernel, grid, dim3(GG_BLOCK), smem,
-                       stream, x, w, offs, out, N, K);
+                       stream, x, w, offs, out, N, K, we, wn);
 }

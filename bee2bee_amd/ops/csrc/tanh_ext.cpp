@@ -1,8 +1,7 @@
 // Torch bindings for the dynamic-tanh stack kernels (tanh_stack.hip).
 // Shapes, strides and dtypes are validated here so the kernels index without
-// checks. Activations are bf16 or fp32; residual, norm weights and routing
-// weights are fp32. All entry points are hipGraph-capture safe (no sync, no
-// host reads).
+// checks. Activations are bf16 or fp32; residual and norm weights are fp32.
+// All entry points are hipGraph-capture safe (no sync, no host reads).
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 #include <hip/hip_runtime.h>
@@ -19,8 +18,6 @@ void launch_proj_norm_store(void*, long, int, const void*, long, const void*,
                             long, int, int, int, const float*, const float*,
                             int, float, float, void*, void*, int, const int*,
                             long, int, int, hipStream_t);
-void launch_routed_silu_glu(const void*, const float*, const int*, void*, long,
-                            int, int, int, int, int, hipStream_t);
 }
 
 namespace {
@@ -148,24 +145,6 @@ void proj_norm_store(Tensor& q, const Tensor& k, const Tensor& v,
         slot_mapping.data_ptr<int>(), T, c, vec ? 1 : 0, stream());
 }
 
-Tensor routed_silu_glu(const Tensor& gu, const Tensor& weights,
-                       const Tensor& idx) {
-    const int c = act_code(gu, "gate_up");
-    check_f32(weights, "weights");
-    check_i32(idx, "idx");
-    TORCH_CHECK(gu.dim() == 3 && gu.is_contiguous() && gu.size(2) % 2 == 0);
-    const long T = gu.size(0);
-    const int E = (int)gu.size(1), I = (int)gu.size(2) / 2;
-    TORCH_CHECK(weights.dim() == 2 && weights.size(0) == T &&
-                idx.sizes() == weights.sizes());
-    Tensor out = torch::empty({T, (long)E * I}, gu.options());
-    const bool vec = I % 4 == 0 && aligned4(gu) && aligned4(out);
-    launch_routed_silu_glu(gu.data_ptr(), weights.data_ptr<float>(),
-                           idx.data_ptr<int>(), out.data_ptr(), T, E, I,
-                           (int)weights.size(1), c, vec ? 1 : 0, stream());
-    return out;
-}
-
 }  // namespace
 
 void register_tanh_ops(pybind11::module_& m) {
@@ -174,6 +153,4 @@ void register_tanh_ops(pybind11::module_& m) {
     m.def("proj_norm_store", &proj_norm_store,
           "q/k norm over the whole projection, value norm; keys and values "
           "to the pages");
-    m.def("routed_silu_glu", &routed_silu_glu,
-          "silu GLU of every expert times the routing weight");
 }

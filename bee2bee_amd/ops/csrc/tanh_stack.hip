@@ -1,11 +1,10 @@
 // Memory-bound kernels of the dynamic-tanh layer stacks
 // (x += n_b(f(n_a(x))), n(x) = tanh(alpha x) * w + b): the norm pair around
-// the fp32 residual update, query/key norms over the whole projection with
-// the key/value page store, and the expert activation of steps whose tokens
-// run through every expert's columns of one product.
+// the fp32 residual update, and query/key norms over the whole projection
+// with the key/value page store.
 //
 // Every kernel is instantiated for bf16 (ushort bits) and fp32 activations;
-// residual, norm weights, statistics and routing weights are fp32 in both.
+// residual, norm weights and statistics are fp32 in both.
 #include "common.h"
 
 namespace {
@@ -176,41 +175,6 @@ proj_norm_store_kernel(T* __restrict__ q, long q_tok, int H,
     }
 }
 
-// --------------------------------------------------- routed gated unit
-// gu [T, E, 2I] (gate | up of every expert) -> out [T, E * I]:
-// silu(gate) * up * weight, the token's routing weight for that expert;
-// zeros, without reading gu, for experts the token did not choose.
-template <typename T, int VEC>
-__global__ void __launch_bounds__(TS_THREADS)
-routed_silu_glu_kernel(const T* __restrict__ gu, const float* __restrict__ wt,
-                       const int* __restrict__ idx, T* __restrict__ out,
-                       int E, int I, int top_k) {
-    const int c = (blockIdx.y * TS_THREADS + threadIdx.x) * VEC;
-    if (c >= E * I) return;         // VEC = 4 only when 4 divides I
-    const long t = blockIdx.x;
-    const int e = c / I, i = c - e * I;
-    float w = 0.f;
-    bool chosen = false;
-    for (int j = 0; j < top_k; ++j)
-        if (idx[t * top_k + j] == e) {
-            w = wt[t * top_k + j];
-            chosen = true;
-        }
-    float y[VEC];
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) y[j] = 0.f;
-    if (chosen) {
-        const T* row = gu + (t * E + e) * 2L * I + i;
-        float g[VEC], u[VEC];
-        ldn<T, VEC>(row, g);
-        ldn<T, VEC>(row + I, u);
-#pragma unroll
-        for (int j = 0; j < VEC; ++j)
-            y[j] = g[j] / (1.f + expf(-g[j])) * u[j] * w;
-    }
-    stn<T, VEC>(out + t * E * (long)I + c, y);
-}
-
 }  // namespace
 
 // ---------------------------------------------------------------- launchers
@@ -258,21 +222,4 @@ extern "C" void launch_proj_norm_store(
     else if (vec) PN_LAUNCH(unsigned short, 4);
     else PN_LAUNCH(unsigned short, 1);
 #undef PN_LAUNCH
-}
-
-extern "C" void launch_routed_silu_glu(const void* gu, const float* wt,
-                                       const int* idx, void* out, long T,
-                                       int E, int I, int top_k, int c,
-                                       int vec, hipStream_t s) {
-    if (T == 0) return;
-    const int per = TS_THREADS * (vec ? 4 : 1);
-    const dim3 grid((unsigned)T, (E * I + per - 1) / per);
-#define RG_LAUNCH(TT, V)                                                      \
-    routed_silu_glu_kernel<TT, V><<<grid, TS_THREADS, 0, s>>>(                \
-        (const TT*)gu, wt, idx, (TT*)out, E, I, top_k)
-    if (c && vec) RG_LAUNCH(float, 4);
-    else if (c) RG_LAUNCH(float, 1);
-    else if (vec) RG_LAUNCH(unsigned short, 4);
-    else RG_LAUNCH(unsigned short, 1);
-#undef RG_LAUNCH
 }

@@ -1259,9 +1259,7 @@ def gelu_erf(x: torch.Tensor) -> torch.Tensor:
 #
 # Mechanisms of stacks whose sublayers are x += n_b(f(n_a(x))) with
 # n(x) = tanh(alpha x) * w + b: the norm pair around the fp32 residual
-# update, query/key norms over the whole projection with the page store, and
-# the expert activation of a step whose tokens run through every expert's
-# columns of one product.
+# update, and query/key norms over the whole projection with the page store.
 
 
 def tanh_norm(x: torch.Tensor, n, out_dtype: torch.dtype) -> torch.Tensor:
@@ -1305,6 +1303,10 @@ def proj_norm_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
     v_cache[blk, :, off] = vn.to(v_cache.dtype)
 
 
+
+# ------------------------------------------------------- routed experts
+
+
 def routed_silu_glu(gu: torch.Tensor, weights: torch.Tensor,
                     idx: torch.Tensor) -> torch.Tensor:
     """gu [T, E, 2I] (gate | up of every expert) -> [T, E * I]: silu(gate) *
@@ -1317,3 +1319,26 @@ def routed_silu_glu(gu: torch.Tensor, weights: torch.Tensor,
     y = torch.nn.functional.silu(g) * u * full[..., None]
     y = torch.where((full != 0)[..., None], y, torch.zeros_like(y))
     return y.to(gu.dtype).view(T, E * (I2 // 2))
+
+
+def moe_sort(idx: torch.Tensor, n_experts: int
+             ) -> Tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
+    """idx [T, k]: the pairs (t, j) in a stable order by expert -> pos
+    [T, k], the pair's row; tok [T * k], each row's token; offs [E + 1], the
+    experts' row ranges."""
+    T, k = idx.shape
+    flat = idx.reshape(-1).long()
+    order = torch.argsort(flat, stable=True)
+    pos = torch.empty_like(order)
+    pos[order] = torch.arange(T * k, device=idx.device)
+    offs = torch.zeros(n_experts + 1, dtype=torch.int32, device=idx.device)
+    offs[1:] = torch.bincount(flat, minlength=n_experts).cumsum(0)
+    i32 = torch.int32
+    return pos.view(T, k).to(i32), (order // k).to(i32), offs
+
+
+def moe_combine(y: torch.Tensor, pos: torch.Tensor, weights: torch.Tensor
+                ) -> torch.Tensor:
+    """out[t] = sum_j weights[t, j] * y[pos[t, j]]."""
+    rows = y[pos.long()].float()                       # [T, k, W]
+    return (rows * weights[..., None]).sum(1).to(y.dtype)

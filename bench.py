@@ -264,6 +264,53 @@ def compare_zevilorn(args) -> None:
                                     device, p_batch, p_len, d_batch, d_len)
 
 
+def compare_tudatar(args) -> None:
+    """Prefill and decode throughput of a Tudatar stack (windowed
+    distance-biased attention / latent attention / per-channel delta rule,
+    routed experts in every layer) beside a Zevilorn stack (the closest
+    family: windowed attention, latent attention, a recurrence, routed
+    experts) and the GQA-attention MoE stack, at equal width, layers, heads,
+    head and expert sizes. The window (4096) covers every context here.
+    Random weights, synthetic prompts, one GPU."""
+    from bee2bee_amd.models.hybrid import (tudatar_layer_cfgs,
+                                           zevilorn_layer_cfgs)
+    from bee2bee_amd.models.spec import (ModelSpec, tudatar_spec,
+                                         zevilorn_spec)
+
+    on_gpu = torch.cuda.is_available()
+    device = "cuda:0" if on_gpu else "cpu"
+    vocab, head_dim = 32000, 128
+    p_batch, p_len = 8, (2048 if on_gpu else 48)
+    d_batch, d_len = (64 if on_gpu else 4), (1024 if on_gpu else 32)
+    for size in args.compare_tudatar.split(","):
+        z = HYBRID_SIZES[size.strip()]
+        W, H, ff, E = z["width"], z["heads"], z["ff"], z["experts"]
+        kv_rank, rot_dim, q_rank, rank = 512, 64, 768, 64
+        if not on_gpu:
+            W, H, head_dim, vocab, ff, E = 64, 4, 16, 256, 32, 4
+            kv_rank, rot_dim, q_rank, rank = 24, 8, 32, 8
+        common = dict(heads=H, kv_heads=max(1, H // 4), dim=head_dim,
+                      window=4096, kv_rank=kv_rank, rot_dim=rot_dim,
+                      q_rank=q_rank, experts=E, top_k=2, expert_ff=ff)
+        base = {"vocab": vocab, "width": W, "norm": {"eps": 1e-6},
+                "max_seq_len": 8192}
+        td = tudatar_spec(f"tudatar-{size}", dict(
+            base, logit_scale=0.5, layers=tudatar_layer_cfgs(
+                6, W, delta_heads=H, delta_kv_heads=H, delta_dim=head_dim,
+                rank=rank, **common)))
+        zv = zevilorn_spec(f"zevilorn-{size}", dict(
+            base, layers=zevilorn_layer_cfgs(6, W, gru_width=W, groups=4,
+                                             keep=2, **common)))
+        dense = ModelSpec(
+            name=f"gqa-moe-{size}", vocab_size=vocab, hidden_size=W,
+            intermediate_size=ff, n_layers=6, n_heads=H,
+            n_kv_heads=max(1, H // 4), head_dim=head_dim, rope_theta=1e6,
+            max_seq_len=8192, n_experts=E, top_k_experts=2)
+        for spec in (td, zv, dense):
+            _measure_prefill_decode(spec, "tudatar-vs-others", size, args,
+                                    device, p_batch, p_len, d_batch, d_len)
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -310,6 +357,15 @@ def main() -> None:
                          "of equal width, layer runs, heads and expert "
                          "sizes, at the comma-separated sizes (s, m, l); "
                          "one JSON line per size and model")
+    ap.add_argument("--compare-tudatar", default=None, metavar="SIZES",
+                    help="instead of the headline run: prefill and decode "
+                         "throughput of the Tudatar stack (windowed "
+                         "distance-biased attention, latent attention, "
+                         "per-channel delta rule, sigmoid-routed experts) "
+                         "beside a Zevilorn stack and a GQA-attention MoE "
+                         "stack of equal width, layers, heads and expert "
+                         "sizes, at the comma-separated sizes (s, m, l); "
+                         "one JSON line per size and model")
     ap.add_argument("--preflight", action="store_true",
                     help="run the scale-run preflight checks (RCCL self-"
                          "test, master endpoint, env, rank wiring) and exit")
@@ -335,6 +391,9 @@ def main() -> None:
         return
     if args.compare_zevilorn:
         compare_zevilorn(args)
+        return
+    if args.compare_tudatar:
+        compare_tudatar(args)
         return
 
     from bee2bee_amd.models.spec import resolve_spec

@@ -31,6 +31,8 @@ ext = CUDAExtension(
         os.path.join(CSRC, "sandwich.hip"),
         os.path.join(CSRC, "gated_ext.cpp"),
         os.path.join(CSRC, "gated.hip"),
+        os.path.join(CSRC, "moe_ext.cpp"),
+        os.path.join(CSRC, "moe.hip"),
         os.path.join(CSRC, "tanh_ext.cpp"),
         os.path.join(CSRC, "tanh_stack.hip"),
     ],

@@ -275,6 +275,39 @@ def forward(cfg: dict, W: Weights, tokens: List[int],
 
 # ----------------------------------------------------- small checkpoints
 
+def make_config(*, kinds=("channel_delta", "attention", "latent_attention",
+                          "attention"), vocab=70, width=22, eps=1e-5,
+                logit_scale=0.6, heads=4, kv_heads=2, dim=6, vdim=5,
+                window=9, scale=0.37, lat_heads=3, lat_dim=5, rot_dim=6,
+                lat_vdim=4, kv_rank=11, q_rank=9, lat_scale=0.4, base=300.0,
+                scaling=True, delta_heads=4, delta_kv=2, delta_dim=7,
+                delta_vdim=6, conv=3, experts=5, top=2, ff=10, rscale=1.7,
+                no_mlp=()) -> dict:
+    sc = {"factor": 3.0, "original": 40, "fast": 4.0, "slow": 1.0}
+    if isinstance(scaling, dict):
+        sc = scaling
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = sc
+    mixers = {
+        "attention": {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                      "vdim": vdim, "scale": scale, "mask": {"size": window}},
+        "latent_attention": {"heads": lat_heads, "dim": lat_dim,
+                             "rot_dim": rot_dim, "vdim": lat_vdim,
+                             "kv_rank": kv_rank, "q_rank": q_rank,
+                             "scale": lat_scale, "rot": rot},
+        "channel_delta": {"heads": delta_heads, "kv_heads": delta_kv,
+                          "dim": delta_dim, "vdim": delta_vdim,
+                          "conv": conv}}
+    mlp = {"kind": "moe", "expert": {"ff": ff},
+           "router": {"experts": experts, "top": top, "scale": rscale}}
+    return {"architecture": "Tudatar", "vocab": vocab, "width": width,
+            "norm": {"eps": eps}, "logit_scale": logit_scale,
+            "layers": [{"type": k, "mixer": dict(mixers[k]),
+                        "mlp": None if i in no_mlp else dict(mlp)}
+                       for i, k in enumerate(kinds)]}
+
+
 def tensor_shapes(cfg: dict, a_rank: int = 5, g_rank: int = 7
                   ) -> Dict[str, tuple]:
     """Checkpoint names and shapes of a config; a_rank / g_rank are the
