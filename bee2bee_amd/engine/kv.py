@@ -18,18 +18,20 @@ the SAME page and slot bookkeeping:
   * head-mixing attention layers: the same two pools, k_cache[i] holding
     rotated unit-norm keys, v_cache[i] the value projection; a layer that
     runs several times (a repeated block) has pools per run;
-  * linear-attention / retention / delta-rule layers: no pages, a recurrent
-    state [n_slots, heads, dim, vdim] fp32 per sequence slot;
+  * linear-attention / retention / delta-rule / state-space layers: no
+    pages, a recurrent state [n_slots, heads, dim, vdim] fp32 per sequence
+    slot (dim: the key size, or the state size of a state-space layer);
   * every layer with a convolution: the last taps-1 conv inputs
     [n_slots, taps-1, channels] per sequence slot (the mixer input for the
-    whole-width conv, the q|k|v projection for a delta mixer's short conv);
+    whole-width conv, the q|k|v projection for a delta mixer's short conv,
+    the x|B|C projection for a state-space mixer's);
   * grouped-query attention with a short convolution on its projected
     q|k|v: the two page pools and the last taps-1 projected rows per slot;
   * grouped-query attention whose values are normed per head: normed when
     cached;
   * an element-wise gated recurrence (minGRU): state [n_slots, width] fp32;
-  * a parallel mixer (attention + delta rule or minGRU side by side) has
-    pages AND state in the same layer.
+  * a parallel mixer (attention + delta rule, minGRU or state-space
+    recurrence side by side) has pages AND state in the same layer.
 A sequence owns one state slot from new_seq to free_seq. Slots and pages
 are handed out again without clearing: the kernels never read state or
 cache rows that precede a sequence's position 0.
@@ -133,10 +135,10 @@ class PagedKV:
                 elif m.kind == "min_gru":
                     rec = torch.zeros(n_slots, m.width, device=dev,
                                       dtype=f32)
-                else:   # lightning / retention / delta: recurrent state
+                else:   # lightning / retention / delta / ssd: state
                     rec = torch.zeros(n_slots, m.heads, m.dim, m.vdim,
                                       device=dev, dtype=f32)
-                    if m.kind == "delta" and m.taps > 1:
+                    if m.kind in ("delta", "ssd") and m.taps > 1:
                         conv = torch.zeros(n_slots, m.taps - 1,
                                            m.conv_channels, device=dev,
                                            dtype=self.dtype)

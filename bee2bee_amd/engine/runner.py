@@ -232,6 +232,10 @@ class Runner:
                     return ops.silu_glu(gu)
                 if ffn.act == "gelu":
                     return ops.gelu_erf(gu)
+                if ffn.act == "relu2":
+                    out = torch.empty_like(gu)
+                    ops.relu2(gu, out)
+                    return out
                 return ops.clamped_glu(gu, ffn.limit, ffn.alpha)
         else:
             E, I, top_k = s.n_experts, s.intermediate_size, s.top_k_experts
@@ -260,6 +264,21 @@ class Runner:
         else:
             weights, idx = ops.moe_topk_gate(logits, top_k)  # [T,k]
         T, H = x.shape
+        if ffn is not None and ffn.weight_input:
+            if ffn.act != "relu2":
+                raise ValueError("routing weights on the experts' inputs "
+                                 "need the relu2 activation")
+            if lw.moe_w_up_cat is not None and \
+                    T <= self.MOE_DENSE_MAX_TOKENS:
+                # every expert's columns, and the shared expert's, as two
+                # plain products; relu(w z)^2 (zero where not chosen) between
+                act = ops.routed_relu2(F.linear(x, lw.moe_w_up_cat), weights,
+                                       idx, E, I)
+                return F.linear(act, lw.moe_w_down_cat)
+            # the input products have no bias and relu(w z)^2 = w^2 relu(z)^2:
+            # a weight on what an expert reads is its square on what it
+            # returns
+            weights = weights * weights
 
         if (lw.moe_w_down_cat is not None and ffn.act == "silu_glu"
                 and T <= self.MOE_DENSE_MAX_TOKENS):
@@ -456,6 +475,9 @@ class Runner:
         key = (dims, base, f64,
                tuple(sorted(scaling.items())) if scaling else None)
         t = self._rope_by_cfg.get(key)
+        if t is None and not dims:      # nothing rotates
+            z = torch.zeros(1, 0, dtype=torch.float32, device=self.device)
+            t = self._rope_by_cfg[key] = (z, z)
         if t is None:
             if scaling and "kind" in scaling:
                 # linear or banded frequency scaling
@@ -500,9 +522,13 @@ class Runner:
                 output_size=T)
         meta = (positions, slot_mapping, cu_seqlens, seq_idx, block_table,
                 state_slots, max_qlen)
-        x = F.embedding(input_ids, W.embed).float()
-        if s.embed_scale != 1.0:
-            x = x * s.embed_scale
+        if s.pos_type == "sinusoid":
+            x = ops.embed_sinusoid(input_ids, W.embed, s.embed_scale,
+                                   positions)
+        else:
+            x = F.embedding(input_ids, W.embed).float()
+            if s.embed_scale != 1.0:
+                x = x * s.embed_scale
         n = s.n_layers
         if s.layer_specs[0].form == "sandwich_w":
             return self._forward_sandwich_w(x, meta)
@@ -510,6 +536,8 @@ class Runner:
             return self._forward_parallel_gated(x, meta)
         if s.layer_specs[0].form == "sandwich_tanh":
             return self._forward_sandwich_tanh(x, meta)
+        if s.layer_specs[0].form == "parallel_scaled":
+            return self._forward_parallel_scaled(x, input_ids, meta)
         if s.layer_specs[0].form == "parallel":
             # x += mixer(h) + ffn(h), h = unit(x) * w: the residual add and
             # the next layer's norm run as one kernel
@@ -782,11 +810,13 @@ class Runner:
         y2 = self._moe_mlp(lw, h, ffn=l.ffn)
         return y1, cols("rg1"), y2, cols("rg2")
 
-    def _gqa_attn_part(self, i: int, m, ns, cols, pre, meta) -> torch.Tensor:
+    def _gqa_attn_part(self, i: int, m, ns, cols, pre, meta, out=None,
+                       out_scale: float = 1.0) -> torch.Tensor:
         """Grouped-query attention of layer run i: optional short conv on
         the projected q|k|v (fp32 out), rotation (or the norm over the whole
-        projection) + page store, attention with the spec's cap / score mix
-        / sink / window / distance bias / head gate."""
+        projection, or per head) + page store, attention with the spec's cap
+        / score mix / sink / window / kept first tokens / distance bias /
+        head gate, times out_scale, into `out` (a column slice) when given."""
         (positions, slot_mapping, cu, seq_idx, block_table, state_slots,
          max_qlen) = meta
         T = positions.shape[0]
@@ -820,6 +850,14 @@ class Runner:
             ops.proj_norm_store(q, k, v, ns.q_norm, ns.k_norm, m.v_norm,
                                 self.spec.rms_eps, m.scale, k_cache, v_cache,
                                 slot_mapping)
+        elif m.head_norm:
+            if m.rope_dims or ns.conv_w is not None:
+                raise ValueError("a norm per head does not combine with a "
+                                 "rotation or a convolution")
+            ops.qk_norm_rope_store(q, k, ns.q_norm, ns.k_norm,
+                                   self.spec.rms_eps, 0, positions, None,
+                                   None, ns.q_mult, k_cache, v_cache,
+                                   slot_mapping, v=v)
         else:
             ops.rope_store(q, k, v, q_out, m.rope_dims,
                            m.rope_layout == "interleaved", positions, cos,
@@ -827,11 +865,14 @@ class Runner:
         sink = None
         if m.zero_sink:
             sink = self._zeros_f32(m.heads)
-        out = torch.empty(T, m.out_size, dtype=self.dtype, device=q.device)
+        if out is None:
+            out = torch.empty(T, m.out_size, dtype=self.dtype,
+                              device=q.device)
         ops.gqa_attn(q_out, k_cache, v_cache, block_table, positions, seq_idx,
                      cu, m.softcap, ns.talk if m.score_mix else None, sink,
                      cols(pre + "g") if m.head_gate else None, m.window, out,
-                     max_qlen, dist=ns.dist)
+                     max_qlen, dist=ns.dist, out_scale=out_scale,
+                     keep_first=m.keep_first)
         return out
 
     def _zeros_f32(self, n: int) -> torch.Tensor:
@@ -882,6 +923,98 @@ class Runner:
                     self.kv.rec_state[i], state_slots, cu, positions, out,
                     max_qlen)
         return out
+
+    # --------------------------------------- scaled parallel-form layers
+
+    def _forward_parallel_scaled(self, x: torch.Tensor,
+                                 input_ids: torch.Tensor, meta
+                                 ) -> torch.Tensor:
+        """x += s1 * mixer(n1(x)) + s2 * ffn(n2(x)), then the side input
+        x += unit(P (gelu(G x) * e)) * w with e the layer's slice of the
+        token's side row. The two scaled adds (which also emit x in the
+        activation type for G) are one kernel; the side norm, its add and
+        both norms of the next layer are another."""
+        s, W = self.spec, self.weights
+        eps, dt, n, d = s.rms_eps, self.dtype, s.n_layers, s.side_dim
+        h1, h2 = ops.add_norm_pair(x, None, None, *W.layers[0].norms, eps, dt)
+        for i in range(n):
+            lw, l = W.layers[i], s.layer_specs[i]
+            y1 = self._scaled_mixer(i, l.mixer, lw, h1, meta)
+            y2, y3 = self._scaled_ffn(l.ffn, lw, h2)
+            xc = ops.scaled_add(x, y1, lw.scales[0], y2, lw.scales[1], y3, dt)
+            g = ops.side_gate(F.linear(xc, lw.side_gate), W.side_embed,
+                              i * d, input_ids)
+            y = F.linear(g, lw.side_proj)
+            nxt = W.layers[i + 1].norms if i + 1 < n else (None, None)
+            h1, h2 = ops.add_norm_pair(x, y, lw.side_norm, *nxt, eps, dt)
+            if self.layer_tap is not None:
+                self.layer_tap(i, x)
+        return x
+
+    def _scaled_mixer(self, i: int, m, lw, h: torch.Tensor, meta
+                      ) -> torch.Tensor:
+        """Mixer of layer i on the normed input h: one input GEMM, the
+        parts' kernels writing column slices of ONE buffer (their result
+        scales folded in), one output GEMM that sums them."""
+        from ..models.hybrid import mixer_parts
+
+        ins, _, outs, n_out = lw.layout
+        proj = F.linear(h, lw.w_in)
+
+        def cols(key):
+            off, n = ins[key]
+            return proj[:, off : off + n]
+
+        if m.kind == "latent_attention":
+            o = self._latent_attn_part(i, m, lw.mix[""], cols, "", meta)
+            return F.linear(o, lw.w_out)
+        exact = n_out == sum(n for _, n in outs.values())
+        buf = (torch.empty if exact else torch.zeros)(
+            h.shape[0], n_out, dtype=self.dtype, device=h.device)
+        for pre, part in mixer_parts(m):
+            off, n = outs[pre]
+            out, ns = buf[:, off : off + n], lw.mix[pre]
+            scale = m.left_scale if pre == "left." else m.right_scale
+            if part.kind == "gqa_attention":
+                self._gqa_attn_part(i, part, ns, cols, pre, meta, out, scale)
+            elif part.kind == "ssd":
+                self._ssd_part(i, part, ns, cols, pre, meta, out, scale)
+            else:
+                raise ValueError(f"unknown mixer part {part.kind!r}")
+        return F.linear(buf, lw.w_out)
+
+    def _scaled_ffn(self, f, lw, h: torch.Tensor):
+        """(feed-forward output, shared expert's output when it was computed
+        on its own); (None, None) without a feed-forward."""
+        if f is None:
+            return None, None
+        if not getattr(f, "n_experts", 0):
+            gu = F.linear(h, lw.w_gate_up, lw.w_gate_up_bias)
+            return F.linear(ops.clamped_glu(gu, f.limit, f.alpha), lw.w_down,
+                            lw.w_down_bias), None
+        y = self._moe_mlp(lw, h, ffn=f)
+        if not f.shared_ff or h.shape[0] <= self.MOE_DENSE_MAX_TOKENS:
+            return y, None
+        z = F.linear(h, lw.w_gate_up)
+        ops.relu2(z, z)
+        return y, F.linear(z, lw.w_down)
+
+    def _ssd_part(self, i, m, ns, cols, pre, meta, out, scale) -> None:
+        """State-space recurrence of layer i: short conv + silu on x|B|C,
+        the scan (step size, decay and skip inside), gate and grouped norm
+        into `out`."""
+        positions, _, cu, seq_idx, _, state_slots, max_qlen = meta
+        conv_state = self.kv.conv_state[i]
+        if conv_state is None:       # a single tap carries nothing
+            conv_state = out.new_empty(0)
+        xbc = ops.short_conv(cols(pre + "xbc"), ns.conv_w, conv_state,
+                             state_slots, cu, seq_idx, positions, True,
+                             bias=ns.conv_b, out_dtype=self.dtype)
+        y = ops.ssd_scan(xbc, cols(pre + "dt"), ns.dt_bias, ns.rate, ns.skip,
+                         m.groups, self.kv.rec_state[i], state_slots, cu,
+                         positions, max_qlen)
+        ops.gated_group_norm(y, cols(pre + "z"), ns.norm, m.norm_groups,
+                             self.spec.rms_eps, out, scale)
 
     # ------------------------------------------------- parallel-form layers
 

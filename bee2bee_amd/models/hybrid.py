@@ -57,6 +57,18 @@ Tudatar config.json keys (dynamic-tanh norms before and after each sublayer):
   channel_delta: mixer.{heads, kv_heads, dim, vdim, conv},
   layers[i].mlp.{kind: moe, expert.ff, router.{experts, top, scale}} (or
   null).
+
+Losivik config.json keys (parallel-form layers with a norm per sublayer, a
+vector scale on each sublayer's result, and a per-token side input after
+them; sinusoidal position vectors join the embedding):
+  architecture, vocab, width, embedding.scale, norm.eps, token_side.dim,
+  layers[i].type in {latent_attention, parallel},
+  latent_attention: mixer.{heads, dim, vdim, kv_rank, scale, mask.size},
+  parallel: mixer.left.{heads, kv_heads, dim, vdim, scale,
+  mask.{size, keep_first}}, mixer.right.{heads, vdim, state, groups, conv,
+  norm_groups}, mixer.{left_scale, right_scale},
+  layers[i].mlp.{kind: dense, ff, limit} | {kind: moe, expert.ff,
+  router.{experts, top}, shared.ff} (or null).
 """
 from __future__ import annotations
 
@@ -92,6 +104,8 @@ class LatentAttnSpec:
     rope_scaling: Optional[Dict[str, float]] = None
 
     kind = "latent_attention"
+
+    # rot_dim 0: no positions in the scores; the cached row is the latent
 
     @property
     def in_sizes(self) -> Tuple[Tuple[str, int], ...]:
@@ -272,6 +286,10 @@ class GqaAttnSpec:
     proj_norm: queries and keys RMS-normed over ALL rows of their projection
     at once (before the split into heads), with a weight per row; v_norm:
     each head's value divided by its root mean square before it is cached.
+    head_norm: each query and key head RMS-normed on its own, with a weight
+    of size dim that all heads share (no rotation, no convolution).
+    keep_first: with a window, the first keep_first positions of the
+    sequence stay visible to every later row.
     distance_bias: a_h ln(1 + b_h (i - j)) is taken off every scaled score,
     a_h and b_h learned per head. bias covers q, k, v and, unless out_bias
     is off, the output projection.
@@ -299,6 +317,8 @@ class GqaAttnSpec:
     v_norm: bool = False
     distance_bias: bool = False
     out_bias: bool = True
+    head_norm: bool = False
+    keep_first: int = 0
 
     kind = "gqa_attention"
 
@@ -342,12 +362,48 @@ class MinGRUSpec:
 
 
 @dataclass
+class SSDSpec:
+    """State-space recurrence with a scalar decay per head and token, and
+    input and read-out vectors shared by groups of heads:
+    S_t = exp(-exp(A_log_h) d) S_(t-1) + d B_t x_t^T, y_t = S_t^T C_t + D_h x_t,
+    d = softplus(dt_t + dt_bias_h). One projection gives [z | x | B | C | dt];
+    x, B and C pass a short causal per-channel convolution with a bias, then
+    silu. The read-out times silu(z) is RMS-normed in norm_groups equal
+    parts, with a weight per channel. State [heads, state, vdim] fp32."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int
+    norm_groups: int = 1
+
+    kind = "ssd"
+
+    @property
+    def dim(self) -> int:
+        return self.state
+
+    @property
+    def conv_channels(self) -> int:
+        return self.out_size + 2 * self.groups * self.state
+
+    @property
+    def in_sizes(self) -> Tuple[Tuple[str, int], ...]:
+        return (("z", self.out_size), ("xbc", self.conv_channels),
+                ("dt", self.heads))
+
+    @property
+    def out_size(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclass
 class ParallelMixerSpec:
     """Two mixers on the same input. combine "scaled_sum": summed with
     fixed scales; "normed_mean": each side's projected output is RMS-normed
     over the model width with a weight of its own, then half their sum."""
     left: Any               # SinkAttnSpec | GqaAttnSpec
-    right: Any              # DeltaSpec | MinGRUSpec
+    right: Any              # DeltaSpec | MinGRUSpec | SSDSpec
     left_scale: float = 1.0
     right_scale: float = 1.0
     combine: str = "scaled_sum"
@@ -367,9 +423,14 @@ class ParallelMixerSpec:
 class DenseFFNSpec:
     """down(act(up h)); act "relu2" is the square of relu; "polynorm" is
     a unit(z) + b unit(z^2) + c unit(z^3) + e with four learned numbers
-    (powers element by element, unit over the ff axis)."""
+    (powers element by element, unit over the ff axis). act "clamped_glu":
+    down(g sigmoid(alpha g) (u + 1)), g = min(gate h, limit), u = clamp(up h,
+    +-limit). bias: every projection has one."""
     ff: int
     act: str = "relu2"
+    limit: float = 0.0
+    alpha: float = 1.702
+    bias: bool = False
 
 
 @dataclass
@@ -387,7 +448,10 @@ class MoEFFNSpec:
     with scores = sigmoid of each logit. group_top: a group's score is the
     sum of its group_top largest expert scores.
     act "gelu": experts without a gate, y = down(gelu(up h)), exact (erf)
-    gelu.
+    gelu. act "relu2": likewise with the square of relu.
+    weight_input: a routing weight multiplies what its expert READS,
+    expert(w h), instead of what it returns; the shared expert has the same
+    form as the others.
     choice_bias: a learned number per expert joins the scores for the choice
     only. renorm: the chosen scores are divided by their sum (+ 1e-20);
     route_scale multiplies the weights last."""
@@ -406,11 +470,12 @@ class MoEFFNSpec:
     choice_bias: bool = False
     renorm: bool = False
     route_scale: float = 1.0
+    weight_input: bool = False
 
     @property
     def up_rows(self) -> int:
         """Rows of one expert's input-side matrix."""
-        return self.ff if self.act == "gelu" else 2 * self.ff
+        return self.ff if self.act in ("gelu", "relu2") else 2 * self.ff
 
 
 @dataclass
@@ -424,6 +489,9 @@ class LayerSpec:
     # tanh(alpha x) * w + b (no row statistics).
     # "parallel_gated": x += sigmoid(W1 h + b1) * mixer(h)
     #                      + sigmoid(W2 h + b2) * ffn(h), h = norm(x) * w.
+    # "parallel_scaled": x += s1 * mixer(h1) + s2 * ffn(h2), h1 and h2 two
+    # weighted norms of the same x, s1 and s2 vectors; then the per-token
+    # side input of ModelSpec.side_dim.
     form: str = "sandwich"
     # layer whose tensors this layer uses (its own cache and state)
     weights_of: Optional[int] = None
@@ -784,6 +852,73 @@ def tanh_layer_specs_from_cfg(layers: List[Dict[str, Any]]
             for i, l in enumerate(layers)]
 
 
+def _losivik_mixer_from_cfg(kind: str, m: Dict[str, Any]):
+    if kind == "latent_attention":
+        return LatentAttnSpec(
+            heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=0,
+            vdim=int(m["vdim"]), kv_rank=int(m["kv_rank"]),
+            window=int((m.get("mask") or {}).get("size", 0) or 0),
+            rope_base=10000.0, rope_dims=0, scale=float(m["scale"]))
+    if kind == "parallel":
+        a, b = m["left"], m["right"]
+        left = _gqa_attn_from_cfg(a, head_norm=True)
+        left.rope_dims = 0          # positions do not enter the scores
+        left.keep_first = int((a.get("mask") or {}).get("keep_first", 0) or 0)
+        right = SSDSpec(
+            heads=int(b["heads"]), vdim=int(b["vdim"]), state=int(b["state"]),
+            groups=int(b.get("groups", 1)), taps=int(b["conv"]),
+            norm_groups=int(b.get("norm_groups", 1)))
+        if right.heads % right.groups:
+            raise ValueError("state space: heads must be a multiple of groups")
+        if right.out_size % right.norm_groups:
+            raise ValueError("state space: norm_groups must divide the "
+                             "inner width")
+        return ParallelMixerSpec(left=left, right=right,
+                                 left_scale=float(m["left_scale"]),
+                                 right_scale=float(m["right_scale"]))
+    raise ValueError(f"unknown mixer type {kind!r}")
+
+
+def _losivik_ffn_from_cfg(f: Optional[Dict[str, Any]]):
+    if not f:
+        return None
+    kind = f.get("kind")
+    if kind == "dense":
+        return DenseFFNSpec(ff=int(f["ff"]), act="clamped_glu",
+                            limit=float(f["limit"]), bias=True)
+    if kind != "moe":
+        raise ValueError(f"unknown feed-forward kind {kind!r}")
+    E, top = int(f["router"]["experts"]), int(f["router"]["top"])
+    if not 1 <= top <= E:
+        raise ValueError("router: top must lie between 1 and experts")
+    return MoEFFNSpec(n_experts=E, top_k=top, ff=int(f["expert"]["ff"]),
+                      shared_ff=int((f.get("shared") or {}).get("ff", 0)),
+                      act="relu2", score="sigmoid_all", weight_input=True)
+
+
+def scaled_layer_specs_from_cfg(layers: List[Dict[str, Any]]
+                                ) -> List[LayerSpec]:
+    """Losivik: a windowed latent attention, or a windowed attention with
+    kept first tokens beside a state-space recurrence; a dense clamped GLU,
+    routed relu^2 experts or no feed-forward."""
+    return [LayerSpec(mixer=_losivik_mixer_from_cfg(l["type"], l["mixer"]),
+                      ffn=_losivik_ffn_from_cfg(l.get("mlp")),
+                      form="parallel_scaled", src=i)
+            for i, l in enumerate(layers)]
+
+
+def mixer_out_layout(l: LayerSpec) -> Tuple[Dict[str, Tuple[int, int]], int]:
+    """Columns of the ONE output matrix of a layer's mixer: the parts'
+    outputs side by side as its K axis, each segment starting on a multiple
+    of 8 elements. Returns ({prefix: (offset, size)}, total)."""
+    outs: Dict[str, Tuple[int, int]] = {}
+    end = 0
+    for pre, m in mixer_parts(l.mixer):
+        outs[pre] = (_pad8(end), m.out_size)
+        end = _pad8(end) + m.out_size
+    return outs, end
+
+
 def mixer_layout(l: LayerSpec) -> Tuple[Dict[str, Tuple[int, int]], int]:
     """Rows of the ONE input matrix of a layer's mixer: every projection
     that reads the mixer input, per part in in_sizes order. Every segment
@@ -890,6 +1025,9 @@ def hybrid_n_params(width: int, vocab: int, taps: int,
         if l.form == "sandwich_tanh":
             n += _tanh_layer_params(width, l, active_only)
             continue
+        if l.form == "parallel_scaled":
+            n += _scaled_layer_params(width, l, active_only)
+            continue
         n += 4 + width * taps
         if m.kind == "latent_attention":
             n += width * (m.q_size + m.cache_dim + m.heads) + m.kv_rank
@@ -935,6 +1073,26 @@ def _tanh_layer_params(width: int, l: LayerSpec, active_only: bool) -> int:
         e = f.top_k if active_only else f.n_experts
         n += 2 * (2 * width + 1) + (width + 1) * f.n_experts
         n += 3 * width * e * f.ff
+    return n
+
+
+def _scaled_layer_params(width: int, l: LayerSpec, active_only: bool) -> int:
+    n = 2 * width
+    for _, m in mixer_parts(l.mixer):
+        n += width * (m.out_size + sum(sz for _, sz in m.in_sizes))
+        if m.kind == "latent_attention":
+            n += m.kv_rank * (1 + m.heads * (m.dim + m.vdim))
+        elif m.kind == "gqa_attention":
+            n += 2 * m.dim
+        else:
+            n += (m.taps + 1) * m.conv_channels + 3 * m.heads + m.out_size
+    f = l.ffn
+    if isinstance(f, DenseFFNSpec):
+        n += 2 * width + 3 * width * f.ff + 2 * f.ff + width
+    elif f is not None:
+        e = f.top_k if active_only else f.n_experts
+        n += 2 * width + width * f.n_experts
+        n += 2 * width * (e * f.ff + f.shared_ff)
     return n
 
 
@@ -1159,4 +1317,43 @@ def tudatar_layer_cfgs(n_layers: int, width: int, *, heads: int = 16,
                      "dim": delta_dim, "vdim": delta_dim, "conv": taps,
                      "decay_rank": rank, "gate_rank": rank}
         out.append({"type": typ, "mixer": mixer, "mlp": mlp})
+    return out
+
+
+def losivik_layer_cfgs(n_layers: int, width: int, *, heads: int = 16,
+                       kv_heads: int = 4, dim: int = 128, window: int = 1024,
+                       keep_first: int = 4, kv_rank: int = 512,
+                       ssd_heads: Optional[int] = None, ssd_vdim: int = 64,
+                       state: int = 128, groups: int = 1, taps: int = 4,
+                       experts: int = 8, top_k: int = 2,
+                       expert_ff: int = 1024, ff: int = 4096
+                       ) -> List[Dict[str, Any]]:
+    """config.json 'layers' entries of a synthetic Losivik stack for
+    benchmarks: latent attention with routed experts and attention beside a
+    state-space recurrence with a dense feed-forward, in turn, every third
+    pair with the feed-forward kinds swapped."""
+    moe = {"kind": "moe", "expert": {"ff": expert_ff},
+           "router": {"experts": experts, "top": top_k},
+           "shared": {"ff": expert_ff}}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    out = []
+    for i in range(n_layers):
+        if i % 2 == 0:
+            typ = "parallel"
+            mixer: Dict[str, Any] = {
+                "left": {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                         "vdim": dim, "scale": dim ** -0.5,
+                         "mask": {"size": window, "keep_first": keep_first}},
+                "right": {"heads": ssd_heads or 2 * width // ssd_vdim,
+                          "vdim": ssd_vdim, "state": state, "groups": groups,
+                          "norm_groups": groups, "conv": taps},
+                "left_scale": 0.75, "right_scale": 0.5}
+        else:
+            typ = "latent_attention"
+            mixer = {"heads": heads, "dim": dim, "vdim": dim,
+                     "kv_rank": kv_rank, "scale": dim ** -0.5,
+                     "mask": {"size": window}}
+        swap = i % 6 >= 4
+        out.append({"type": typ, "mixer": mixer,
+                    "mlp": dense if (i % 2 == 0) != swap else moe})
     return out

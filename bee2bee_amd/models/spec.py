@@ -38,7 +38,9 @@ class ModelSpec:
     arch: str = "llama"          # "llama" | "gpt2" (HF weight mapping)
     norm_type: str = "rmsnorm"   # "rmsnorm" | "layernorm"
     act_type: str = "swiglu"     # "swiglu" | "gelu" (gelu: fc -> act -> proj)
-    pos_type: str = "rope"       # "rope" | "learned"
+    # "rope" | "learned" | "sinusoid" (fixed sin/cos vectors added to the
+    # embedding) | "none"
+    pos_type: str = "rope"
     attn_out_bias: bool = False
     mlp_bias: bool = False
     # llama3-type RoPE scaling (Llama-3.1/3.2 checkpoints):
@@ -49,7 +51,8 @@ class ModelSpec:
     bos_token_id: int = 1
     eos_token_id: int = 2
     # hybrid stacks (arch "nukopel", "pugozen", "pimodra", "zevilorn",
-    # "tudatar"): per-layer mixer/feed-forward specs (models/hybrid.py). When set, the uniform-layer fields above hold
+    # "tudatar", "losivik"): per-layer mixer/feed-forward specs
+    # (models/hybrid.py). When set, the uniform-layer fields above hold
     # representative maxima only; the Runner's hybrid path reads these.
     layer_specs: Optional[List[Any]] = None
     embed_scale: float = 1.0     # x = embed[token] * embed_scale
@@ -57,6 +60,7 @@ class ModelSpec:
     norm_groups: int = 1         # weighted RMS norms over equal parts of a row
     step_rows: int = 0           # rows of the per-pass residual step table
     logit_scale: float = 1.0     # logits = head(norm(x)) * logit_scale
+    side_dim: int = 0            # per-token side input of every layer
     # the config.json "layers" / "loop" entries a looped stack was unrolled
     # from (kept for export)
     source_cfg: Optional[Dict[str, Any]] = None
@@ -82,8 +86,9 @@ class ModelSpec:
         if self.is_hybrid:
             from .hybrid import hybrid_n_params
 
-            return hybrid_n_params(self.hidden_size, self.vocab_size,
-                                   self.canon_taps, self.layer_specs)
+            return self._side_params() + hybrid_n_params(
+                self.hidden_size, self.vocab_size, self.canon_taps,
+                self.layer_specs)
         h, i = self.hidden_size, self.intermediate_size
         attn = h * (self.q_size + 2 * self.kv_size) + self.q_size * h
         if self.is_moe:
@@ -98,14 +103,23 @@ class ModelSpec:
         head = 0 if self.tie_embeddings else self.vocab_size * h
         return emb + self.n_layers * per_layer + head + h
 
+    def _side_params(self) -> int:
+        """Side-input tables and projections; a stack that has them ties its
+        output matrix to the embedding (hybrid_n_params counts two)."""
+        if not self.side_dim:
+            return 0
+        W, V, L, d = (self.hidden_size, self.vocab_size, self.n_layers,
+                      self.side_dim)
+        return L * d * (V + 2 * W) + L * W - (V - 1) * W - 1
+
     def active_params_per_token(self) -> int:
         """Params touched per decoded token (MoE: only top-k experts)."""
         if self.is_hybrid:
             from .hybrid import hybrid_n_params
 
-            return hybrid_n_params(self.hidden_size, self.vocab_size,
-                                   self.canon_taps, self.layer_specs,
-                                   active_only=True)
+            return self._side_params() + hybrid_n_params(
+                self.hidden_size, self.vocab_size, self.canon_taps,
+                self.layer_specs, active_only=True)
         if not self.is_moe:
             return self.n_params()
         h, i = self.hidden_size, self.intermediate_size
@@ -547,6 +561,31 @@ def tudatar_spec(name: str, cfg: Dict[str, Any],
     return spec
 
 
+def losivik_spec(name: str, cfg: Dict[str, Any]) -> ModelSpec:
+    """Parse a Losivik config.json dict: parallel-form layers with two norms
+    and a vector scale per sublayer, a latent attention or an attention
+    beside a state-space recurrence, dense or routed feed-forwards, a
+    per-token side input after every layer, sinusoidal positions, tied
+    output embedding."""
+    from .hybrid import mixer_parts, scaled_layer_specs_from_cfg
+
+    layers = scaled_layer_specs_from_cfg(cfg["layers"])
+    spec = hybrid_spec(
+        name, int(cfg["vocab"]), int(cfg["width"]), layers,
+        eps=float(cfg["norm"]["eps"]),
+        embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+        canon_taps=0, max_seq_len=int(cfg.get("max_seq_len", 32768)),
+        arch="losivik", norm_type="rmsnorm", act_type="clamped_glu",
+    )
+    spec.tie_embeddings = True
+    spec.pos_type = "sinusoid"
+    spec.side_dim = int(cfg["token_side"]["dim"])
+    spec.n_kv_heads = max(getattr(m, "kv_heads", 1) for l in layers
+                          for _, m in mixer_parts(l.mixer))
+    spec.source_cfg = {"layers": cfg["layers"]}
+    return spec
+
+
 def resolve_spec(name: str, model_path: Optional[str] = None) -> ModelSpec:
     """Resolve a model name (preset / alias / HF id / local dir) to a spec.
 
@@ -603,6 +642,9 @@ def spec_from_hf_config(model_path: str, name: Optional[str] = None) -> ModelSpe
         return tudatar_spec(
             name or os.path.basename(os.path.normpath(model_path)), cfg,
             safetensors_shapes(model_path))
+    if cfg.get("architecture") == "Losivik":
+        return losivik_spec(
+            name or os.path.basename(os.path.normpath(model_path)), cfg)
     if cfg.get("model_type") == "gpt2" or "n_embd" in cfg:
         spec = _gpt2(
             name or cfg.get("_name_or_path", os.path.basename(model_path)),

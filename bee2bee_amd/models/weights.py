@@ -51,6 +51,11 @@ class LayerWeights:
         # routed experts: a number per expert added to the scores for the
         # choice; the experts' output matrices side by side [W, E * ff]
         "moe_choice_bias", "moe_w_down_cat",
+        # the input matrix of every expert and the shared one [E*ff + sh, W]
+        "moe_w_up_cat",
+        # parallel-form layers with scaled sublayers and a side input: the
+        # two result scales, the side projections and its norm weight
+        "scales", "side_gate", "side_proj", "side_norm",
     )
 
     def __init__(self) -> None:
@@ -87,7 +92,12 @@ class LayerWeights:
         self.act_coef = None   # [4] fp32 (PolyNorm a, b, c, e)
         self.b_in = None       # [in_total] (zeros where a part has no bias)
         self.moe_choice_bias = None   # [E] fp32
-        self.moe_w_down_cat = None    # [width, E * ff]
+        self.moe_w_down_cat = None    # [width, E * ff [+ shared ff]]
+        self.moe_w_up_cat = None      # [E * ff [+ shared ff], width]
+        self.scales = None     # (mixer, ffn or None): [width] fp32 each
+        self.side_gate = None  # [side_dim, width]
+        self.side_proj = None  # [width, side_dim]
+        self.side_norm = None  # [width] fp32
 
 
 class ModelWeights:
@@ -106,6 +116,8 @@ class ModelWeights:
         self.final_tanh: Optional[Tuple] = None
         self.final_tanh_scaled: Optional[Tuple] = None
         self.step_table: Optional[torch.Tensor] = None  # [passes, hidden] fp32
+        # per-token side input table [vocab, n_layers * side_dim]
+        self.side_embed: Optional[torch.Tensor] = None
         self.layers = [LayerWeights() for _ in range(spec.n_layers)]
         # expert-parallel shard: when set, MoE expert tensors hold only
         # experts [lo, hi) (gate stays replicated); see parallel/ep.py
@@ -141,6 +153,8 @@ class ModelWeights:
                 return self._random_init_zevilorn(seed)
             if s.arch == "tudatar":
                 return self._random_init_tudatar(seed)
+            if s.arch == "losivik":
+                return self._random_init_losivik(seed)
             return self._random_init_hybrid(seed)
         lo, hi = layer_range or (0, s.n_layers)
         self.expert_range = expert_range
@@ -246,6 +260,8 @@ class ModelWeights:
                 return self._load_zevilorn(model_path)
             if s.arch == "tudatar":
                 return self._load_tudatar(model_path)
+            if s.arch == "losivik":
+                return self._load_losivik(model_path)
             return self._load_nukopel(model_path)
         if s.arch == "gpt2":
             return self._load_gpt2(model_path, layer_range)
@@ -725,7 +741,7 @@ class ModelWeights:
         ns.conv_w = self._conv_taps(q, get) if m.taps else None
         ns.talk = self._f32(get(q + "talk")) if m.score_mix else None
         ns.q_norm = ns.k_norm = ns.dist = None
-        if m.proj_norm:
+        if m.proj_norm or m.head_norm:
             ns.q_norm = self._f32(get(q + "q.norm"))
             ns.k_norm = self._f32(get(q + "k.norm"))
         if m.distance_bias:
@@ -750,6 +766,20 @@ class ModelWeights:
             m.heads, m.vdim, m.kv_rank).transpose(1, 2))
         ns.sink = self._f32(get(q + "sink")) if m.sink else None
         ns.wo_b = None
+
+    def _mix_ssd(self, ns, m, pre: str, q: str, get, put_in) -> None:
+        rows, at = get(q + "in"), 0
+        for name, n in m.in_sizes:
+            put_in(pre + name, rows[at : at + n])
+            at += n
+        # checkpoint [channels, taps] -> tap-major [taps, channels]
+        ns.conv_w = self._f32(get(q + "conv").t())
+        ns.conv_b = self._f32(get(q + "conv.b"))
+        # decay rate exp(A_log), evaluated once in fp32
+        ns.rate = torch.exp(self._f32(get(q + "A_log")))
+        ns.dt_bias = self._f32(get(q + "dt_bias"))
+        ns.skip = self._f32(get(q + "D"))
+        ns.norm = self._f32(get(q + "norm"))
 
     def _mix_delta(self, ns, m, pre: str, q: str, get, put_in) -> None:
         put_in(pre + "qkv", torch.cat(
@@ -814,6 +844,16 @@ class ModelWeights:
         else:
             table["g"] = ((H * Dv, W), 0.0, lin)
         return table
+
+    @staticmethod
+    def _ssd_shapes(m, W: int) -> Dict[str, tuple]:
+        """{tensor: (shape, init mean, init std)} of a state-space mixer."""
+        ch = m.conv_channels
+        return {"in": ((sum(n for _, n in m.in_sizes), W), 0.0, W ** -0.5),
+                "conv": ((ch, m.taps), 0.0, 0.4), "conv.b": ((ch,), 0.0, 0.1),
+                "dt_bias": ((m.heads,), -3.0, 0.5),
+                "A_log": ((m.heads,), 0.5, 0.5), "D": ((m.heads,), 1.0, 0.1),
+                "norm": ((m.out_size,), 1.0, 0.1)}
 
     # ------------------------------------------------ dynamic-tanh stacks
 
@@ -946,6 +986,164 @@ class ModelWeights:
                 get(f"{p}mlp.e{e}.down") for e in range(f.n_experts)], dim=1))
             lw.moe_w_down = lw.moe_w_down_cat.view(
                 W, f.n_experts, f.ff).permute(1, 0, 2)
+
+    # ------------------------------------------- scaled parallel-form stacks
+
+    @torch.no_grad()
+    def _load_losivik(self, model_path: str) -> "ModelWeights":
+        """Losivik safetensors: 'embed' (also the output matrix),
+        'side.embed' [vocab, layers * side dim], 'final.norm' and per layer
+        'l<i>.norm1|norm2' (norm weights, stored as the difference from 1),
+        'l<i>.ls1|ls2', 'l<i>.mix.*' ('.left.*' / '.right.*' for a parallel
+        mixer), 'l<i>.mlp.gate|up|down' + '.b' (dense) or
+        'l<i>.mlp.router|e<k>.up|down|shared.up|down' (experts) and
+        'l<i>.side.gate|proj|norm'. Linear weights [out, in]."""
+        tensors = dict(iter_safetensors(model_path))
+        self._assemble_losivik(lambda name: tensors.pop(name))
+        return self
+
+    @torch.no_grad()
+    def _random_init_losivik(self, seed: int) -> "ModelWeights":
+        import zlib
+
+        def get(name: str) -> torch.Tensor:
+            tseed = (seed * 1000003 + zlib.crc32(name.encode())) % (2**31)
+            gen = torch.Generator(device=self.device).manual_seed(tseed)
+            shape, mean, std = self._losivik_shape(name)
+            t = torch.randn(tuple(shape), generator=gen, dtype=torch.float32,
+                            device=self.device)
+            return (mean + std * t).bfloat16()
+
+        self._assemble_losivik(get)
+        return self
+
+    def _losivik_shape(self, name: str):
+        """(shape, init mean, init std) of a checkpoint tensor."""
+        s = self.spec
+        W, V, d = s.hidden_size, s.vocab_size, s.side_dim
+        lin = W ** -0.5
+        if name == "embed":
+            return (V, W), 0.0, lin
+        if name == "side.embed":
+            return (V, s.n_layers * d), 0.0, 1.0
+        head, rest = name.split(".", 1)
+        if head == "final" or rest in ("norm1", "norm2"):
+            return (W,), 0.0, 0.1
+        if rest in ("ls1", "ls2"):
+            return (W,), 0.5, 0.1
+        if rest.startswith("side."):
+            return {"gate": ((d, W), 0.0, lin), "proj": ((W, d), 0.0, d ** -0.5),
+                    "norm": ((W,), 0.2, 0.05)}[rest[len("side."):]]
+        l = s.layer_specs[int(head[1:])]
+        m, f = l.mixer, l.ffn
+        if rest.startswith("mlp."):
+            rest = rest[len("mlp."):]
+            if rest == "router":
+                return (f.n_experts, W), 0.0, lin
+            ff = f.shared_ff if rest.startswith("shared.") else f.ff
+            if rest.endswith(".b"):
+                return (W if rest.startswith("down") else ff,), 0.0, 0.1
+            if rest.endswith("down"):
+                return (W, ff), 0.0, ff ** -0.5
+            return (ff, W), 0.0, lin
+        rest = rest[len("mix."):]
+        if m.kind == "parallel":
+            side, rest = rest.split(".", 1)
+            m = m.left if side == "left" else m.right
+        if rest == "o":
+            return (W, m.out_size), 0.0, m.out_size ** -0.5
+        if m.kind == "latent_attention":
+            return self._latent_shapes(m, W)[rest]
+        if m.kind == "ssd":
+            return self._ssd_shapes(m, W)[rest]
+        if rest.endswith(".norm"):
+            return (m.dim,), 1.0, 0.1
+        return (dict(m.in_sizes)[rest], W), 0.0, lin
+
+    def _assemble_losivik(self, get) -> None:
+        """Engine layout of a scaled parallel-form stack: per layer ONE input
+        matrix for the mixer (models/hybrid.py mixer_layout) and ONE output
+        matrix with the parts' K axes side by side (mixer_out_layout); norm
+        weights as 1 + w in fp32; gate|up of a dense feed-forward as one
+        matrix with its bias; experts' (and the shared expert's) input and
+        output matrices each as one matrix, so a step with few tokens runs
+        them as two products. `moe_w_gate_up`, `moe_w_down`, `w_gate_up` and
+        `w_down` are its views per expert and for the shared one."""
+        from types import SimpleNamespace
+
+        from .hybrid import mixer_layout, mixer_out_layout, mixer_parts
+
+        s = self.spec
+        W = s.hidden_size
+
+        def norm(name: str) -> torch.Tensor:
+            return 1.0 + self._f32(get(name))
+
+        self.embed = self._act(get("embed"))
+        self.lm_head = self.embed
+        self.side_embed = self._act(get("side.embed"))
+        self.final_norm = norm("final.norm")
+        for i, l in enumerate(s.layer_specs):
+            lw, p, f = self.layers[i], f"l{i}.", l.ffn
+            ins, n_in = mixer_layout(l)
+            outs, n_out = mixer_out_layout(l)
+            lw.layout = (ins, n_in, outs, n_out)
+            lw.norms = (norm(p + "norm1"),
+                        norm(p + "norm2") if f is not None else None)
+            lw.scales = (self._f32(get(p + "ls1")),
+                         self._f32(get(p + "ls2")) if f is not None else None)
+            w_in = torch.zeros(n_in, W, device=self.device, dtype=self.dtype)
+            w_out = torch.zeros(W, n_out, device=self.device,
+                                dtype=self.dtype)
+
+            def put_in(key: str, t, bias: bool = False) -> None:
+                off, n = ins[key]
+                name, t = (t, get(t)) if isinstance(t, str) else (key, t)
+                assert t.shape == (n, W), (name, tuple(t.shape), n)
+                w_in[off : off + n] = t.to(self.device, self.dtype)
+
+            lw.mix = {}
+            for pre, m in mixer_parts(l.mixer):
+                ns = lw.mix[pre] = SimpleNamespace()
+                mix = {"gqa_attention": self._mix_gqa, "ssd": self._mix_ssd,
+                       "latent_attention": self._mix_latent}[m.kind]
+                mix(ns, m, pre, p + "mix." + pre, get, put_in)
+                if m.kind == "gqa_attention":
+                    # per-head score multiplier folded into the query norm
+                    ns.q_mult = torch.full((m.heads,), m.scale,
+                                           dtype=torch.float32,
+                                           device=self.device)
+                off, n = outs[pre]
+                w_out[:, off : off + n] = get(p + "mix." + pre + "o").to(
+                    self.device, self.dtype)
+            lw.w_in, lw.w_out = w_in, w_out
+            lw.side_gate = self._act(get(p + "side.gate"))
+            lw.side_proj = self._act(get(p + "side.proj"))
+            lw.side_norm = self._f32(get(p + "side.norm"))
+            if f is None:
+                continue
+            q = p + "mlp."
+            if not getattr(f, "n_experts", 0):
+                lw.w_gate_up = self._act(torch.cat([get(q + "gate"),
+                                                    get(q + "up")]))
+                lw.w_gate_up_bias = self._act(torch.cat([get(q + "gate.b"),
+                                                         get(q + "up.b")]))
+                lw.w_down = self._act(get(q + "down"))
+                lw.w_down_bias = self._act(get(q + "down.b"))
+                continue
+            E, n = f.n_experts, f.n_experts * f.ff
+            parts = [f"e{e}." for e in range(E)] +                 (["shared."] if f.shared_ff else [])
+            lw.moe_gate = self._f32(get(q + "router"))
+            lw.moe_w_up_cat = self._act(torch.cat(
+                [get(q + k + "up") for k in parts]))
+            lw.moe_w_down_cat = self._act(torch.cat(
+                [get(q + k + "down") for k in parts], dim=1))
+            lw.moe_w_gate_up = lw.moe_w_up_cat[:n].view(E, f.ff, W)
+            lw.moe_w_down = lw.moe_w_down_cat[:, :n].unflatten(
+                1, (E, f.ff)).permute(1, 0, 2)
+            if f.shared_ff:
+                lw.w_gate_up = lw.moe_w_up_cat[n:]
+                lw.w_down = lw.moe_w_down_cat[:, n:]
 
     # --------------------------------------------- gated parallel-form stacks
 
@@ -1481,6 +1679,89 @@ def _save_tudatar(weights: "ModelWeights", out_dir: str, tensors, cpu) -> None:
         json.dump(tudatar_config(s), fh, indent=1)
 
 
+def losivik_config(spec: ModelSpec) -> Dict:
+    """The config.json dict of a Losivik spec (inverse of losivik_spec): the
+    layer entries are kept as they were parsed."""
+    return {"architecture": "Losivik", "vocab": spec.vocab_size,
+            "width": spec.hidden_size, "max_seq_len": spec.max_seq_len,
+            "embedding": {"scale": spec.embed_scale},
+            "norm": {"eps": spec.rms_eps}, "token_side": {"dim": spec.side_dim},
+            "layers": (spec.source_cfg or {}).get("layers", [])}
+
+
+def _save_losivik(weights: "ModelWeights", out_dir: str, tensors, cpu) -> None:
+    from safetensors.torch import save_file
+
+    from .hybrid import mixer_parts
+
+    s = weights.spec
+
+    def put(name: str, t: torch.Tensor) -> None:
+        tensors[name] = cpu(t).to(torch.bfloat16).clone()
+
+    put("embed", weights.embed)
+    put("side.embed", weights.side_embed)
+    put("final.norm", weights.final_norm - 1.0)
+    for i, l in enumerate(s.layer_specs):
+        lw, p, f = weights.layers[i], f"l{i}.", l.ffn
+        ins, _, outs, _ = lw.layout
+        for j in (0, 1) if f is not None else (0,):
+            put(f"{p}norm{j + 1}", lw.norms[j] - 1.0)
+            put(f"{p}ls{j + 1}", lw.scales[j])
+        for n_, t in (("gate", lw.side_gate), ("proj", lw.side_proj),
+                      ("norm", lw.side_norm)):
+            put(f"{p}side.{n_}", t)
+        for pre, m in mixer_parts(l.mixer):
+            ns, q = lw.mix[pre], p + "mix." + pre
+
+            def rows(key: str) -> torch.Tensor:
+                off, n = ins[pre + key]
+                return lw.w_in[off : off + n]
+
+            off, n = outs[pre]
+            put(q + "o", lw.w_out[:, off : off + n])
+            if m.kind == "gqa_attention":
+                for n_ in ("q", "k", "v"):
+                    put(q + n_, rows(n_))
+                put(q + "q.norm", ns.q_norm)
+                put(q + "k.norm", ns.k_norm)
+            elif m.kind == "latent_attention":
+                for n_ in ("q", "dkv", "g"):
+                    put(q + n_, rows(n_))
+                put(q + "dkv.norm", ns.kv_norm)
+                put(q + "uk", ns.w_uk.reshape(m.heads * m.dim, m.kv_rank))
+                put(q + "uv", ns.w_uv.transpose(1, 2).reshape(
+                    m.heads * m.vdim, m.kv_rank))
+            else:
+                put(q + "in", torch.cat([rows(k) for k, _ in m.in_sizes]))
+                put(q + "conv", ns.conv_w.t())
+                put(q + "conv.b", ns.conv_b)
+                put(q + "A_log", torch.log(ns.rate))
+                put(q + "dt_bias", ns.dt_bias)
+                put(q + "D", ns.skip)
+                put(q + "norm", ns.norm)
+        if f is None:
+            continue
+        q = p + "mlp."
+        if not getattr(f, "n_experts", 0):
+            for n_, t in (("", (lw.w_gate_up, lw.w_down)),
+                          (".b", (lw.w_gate_up_bias, lw.w_down_bias))):
+                put(q + "gate" + n_, t[0][: f.ff])
+                put(q + "up" + n_, t[0][f.ff :])
+                put(q + "down" + n_, t[1])
+            continue
+        put(q + "router", lw.moe_gate)
+        for e in range(f.n_experts):
+            put(f"{q}e{e}.up", lw.moe_w_gate_up[e])
+            put(f"{q}e{e}.down", lw.moe_w_down[e])
+        if f.shared_ff:
+            put(q + "shared.up", lw.w_gate_up)
+            put(q + "shared.down", lw.w_down)
+    save_file(tensors, os.path.join(out_dir, "model.safetensors"))
+    with open(os.path.join(out_dir, "config.json"), "w") as fh:
+        json.dump(losivik_config(s), fh, indent=1)
+
+
 def safetensors_shapes(model_path: str) -> Dict[str, Tuple[int, ...]]:
     """Tensor name -> shape from the shards' headers (8-byte little-endian
     length, then that many bytes of JSON); no tensor data is read."""
@@ -1778,6 +2059,8 @@ def save_hf(weights: ModelWeights, out_dir: str) -> None:
             _save_zevilorn(weights, out_dir, tensors, cpu)
         elif s.arch == "tudatar":
             _save_tudatar(weights, out_dir, tensors, cpu)
+        elif s.arch == "losivik":
+            _save_losivik(weights, out_dir, tensors, cpu)
         else:
             _save_nukopel(weights, out_dir, tensors, cpu)
         return

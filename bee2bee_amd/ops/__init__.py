@@ -353,15 +353,16 @@ def relu2(x, out) -> None:
 
 def qk_norm_rope_store(q, k, q_norm, k_norm, eps: float, rope_dims: int,
                        positions, cos, sin, q_mult, k_cache, v_cache,
-                       slot_mapping) -> None:
+                       slot_mapping, v=None) -> None:
+    """v None: the values are the keys as projected."""
     if _use_hip(q):
         require_hip().qk_norm_rope_store(q, k, q_norm, k_norm, eps, rope_dims,
                                          positions, cos, sin, q_mult, k_cache,
-                                         v_cache, slot_mapping)
+                                         v_cache, slot_mapping, v)
         return
     reference.qk_norm_rope_store(q, k, q_norm, k_norm, eps, rope_dims,
                                  positions, cos, sin, q_mult, k_cache,
-                                 v_cache, slot_mapping)
+                                 v_cache, slot_mapping, v)
 
 
 def sink_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
@@ -377,12 +378,13 @@ def sink_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
 
 
 def short_conv(x, w, state, state_slots, cu_seqlens, seq_idx, positions,
-               silu: bool = True):
+               silu: bool = True, bias=None, out_dtype=torch.float32):
     if _use_hip(x):
         return require_hip().short_conv(x, w, state, state_slots, cu_seqlens,
-                                        seq_idx, positions, silu)
+                                        seq_idx, positions, silu, bias,
+                                        out_dtype)
     return reference.short_conv(x, w, state, state_slots, cu_seqlens, seq_idx,
-                                positions, silu)
+                                positions, silu, bias, out_dtype)
 
 
 def delta_gates(qk, n_qk_heads: int, dim: int, b, a, dt_bias, rate,
@@ -522,10 +524,13 @@ def rope_store(q, k, v, q_out, rope_dims: int, interleaved: bool, positions,
 
 def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
              cu_seqlens, softcap: float, talk, sink, head_gate, window: int,
-             out, max_qlen: int = 0, dist=None) -> None:
+             out, max_qlen: int = 0, dist=None, out_scale: float = 1.0,
+             keep_first: int = 0) -> None:
     """max_qlen: longest chunk of the step (host int). dist fp32 [2, H]: a
-    logarithmic distance bias on the scores (not together with a cap or a
-    score mix). Without a cap and a
+    logarithmic distance bias on the scores; keep_first: the sequence's
+    first positions stay visible past the window; out_scale multiplies the
+    result (none of the three together with a cap or a score mix). Without
+    a cap and a
     score mix the step runs on the sink-attention kernels; with them, on
     the score-mixing kernels. Both take bf16 prompt portions with head size
     64/128 to the matrix cores."""
@@ -533,12 +538,13 @@ def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
         if talk is None and not softcap:
             require_hip().sink_attn(q, k_cache, v_cache, block_table,
                                     positions, seq_idx, cu_seqlens, sink,
-                                    window, out, 1.0, max_qlen, head_gate,
-                                    dist)
+                                    window, out, float(out_scale), max_qlen,
+                                    head_gate, dist, keep_first)
         else:
-            if dist is not None:
-                raise ValueError("a distance bias does not combine with a "
-                                 "score cap or mix")
+            if dist is not None or keep_first or out_scale != 1.0:
+                raise ValueError("a distance bias, kept first tokens and an "
+                                 "output scale do not combine with a score "
+                                 "cap or mix")
             if talk is None:    # a cap alone: mix with the identity
                 talk = torch.eye(q.shape[1], dtype=torch.float32,
                                  device=q.device)
@@ -549,7 +555,7 @@ def gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
         return
     reference.gqa_attn(q, k_cache, v_cache, block_table, positions, seq_idx,
                        cu_seqlens, softcap, talk, sink, head_gate, window, out,
-                       dist)
+                       dist, out_scale, keep_first)
 
 
 def min_gru(z, x, g, state, state_slots, cu_seqlens, positions, out,
@@ -617,8 +623,79 @@ def proj_norm_store(q, k, v, q_norm, k_norm, v_unit: bool, eps: float,
                               k_cache, v_cache, slot_mapping)
 
 
+# --------------------------------------------- scaled parallel-form stacks
+# (ops/reference.py documents shapes and formulas)
+
+_inv_freq = {}
+
+
+def embed_sinusoid(ids, table, scale: float, positions):
+    """fp32 rows table[id] * scale + the position's sin/cos vector."""
+    W = table.shape[1]
+    key = (W, table.device)
+    f = _inv_freq.get(key)
+    if f is None:
+        f = _inv_freq[key] = reference.sinusoid_freqs(W, table.device)
+    if _use_hip(table):
+        return require_hip().embed_sinusoid(ids, table, float(scale),
+                                            positions, f)
+    return reference.embed_sinusoid(ids, table, scale, positions, f)
+
+
+def add_norm_pair(resid, y, w_post, wa, wb, eps: float, out_dtype):
+    """resid(fp32) += unit(y) * w_post in place (when y is given); -> (unit(
+    resid) * wa, unit(resid) * wb), None for a weight that is None. One pass
+    on the GPU."""
+    if _use_hip(resid):
+        return tuple(require_hip().add_norm_pair(resid, y, w_post, wa, wb,
+                                                 eps, out_dtype))
+    return reference.add_norm_pair(resid, y, w_post, wa, wb, eps, out_dtype)
+
+
+def scaled_add(resid, y1, s1, y2, s2, y3, out_dtype):
+    """resid(fp32) += s1 * y1 [+ s2 * (y2 [+ y3])] in place; -> resid in
+    out_dtype (resid itself when that is fp32)."""
+    if _use_hip(resid):
+        return require_hip().scaled_add(resid, y1, s1, y2, s2, y3, out_dtype)
+    return reference.scaled_add(resid, y1, s1, y2, s2, y3, out_dtype)
+
+
+def side_gate(g, table, offset: int, ids):
+    """gelu_tanh(g) * table[ids, offset : offset + width of g]."""
+    if _use_hip(g):
+        return require_hip().side_gate(g, table, offset, ids)
+    return reference.side_gate(g, table, offset, ids)
+
+
+def ssd_scan(xbc, dt, dt_bias, rate, skip, groups: int, state, state_slots,
+             cu_seqlens, positions, max_qlen: int = 0):
+    """max_qlen: longest chunk of the step (host int); long chunks take the
+    chunk-parallel kernels, short ones and decode rows the token-serial
+    one."""
+    if _use_hip(xbc):
+        return require_hip().ssd_scan(xbc, dt, dt_bias, rate, skip, groups,
+                                      state, state_slots, cu_seqlens,
+                                      positions, max_qlen)
+    return reference.ssd_scan(xbc, dt, dt_bias, rate, skip, groups, state,
+                              state_slots, cu_seqlens, positions)
+
+
+def gated_group_norm(y, z, w, groups: int, eps: float, out,
+                     out_scale: float) -> None:
+    if _use_hip(y):
+        require_hip().gated_group_norm(y, z, w, groups, eps, out,
+                                       float(out_scale))
+        return
+    reference.gated_group_norm(y, z, w, groups, eps, out, out_scale)
+
 
 # ------------------------------------------------------- routed experts
+
+
+def routed_relu2(z, weights, idx, n_experts: int, ff: int):
+    if _use_hip(z):
+        return require_hip().routed_relu2(z, weights, idx, n_experts, ff)
+    return reference.routed_relu2(z, weights, idx, n_experts, ff)
 
 
 def routed_silu_glu(gu, weights, idx):

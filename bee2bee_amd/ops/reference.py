@@ -589,12 +589,12 @@ def qk_norm_rope_store(q: torch.Tensor, k: torch.Tensor, q_norm: torch.Tensor,
                        k_norm: torch.Tensor, eps: float, rope_dims: int,
                        positions: torch.Tensor, cos, sin,
                        q_mult: torch.Tensor, k_cache: torch.Tensor,
-                       v_cache: torch.Tensor,
-                       slot_mapping: torch.Tensor) -> None:
+                       v_cache: torch.Tensor, slot_mapping: torch.Tensor,
+                       v: Optional[torch.Tensor] = None) -> None:
     """q [T, H, D] (view, rewritten in place): rotate(unit(q) * q_norm) *
     q_mult[h]. k [T, G, D] (view, left as is): rotate(unit(k) * k_norm) goes
-    to k_cache, k itself (the value) to v_cache, both
-    [n_blocks, G, block, D] at slot_mapping."""
+    to k_cache [n_blocks, G, block, D], v [T, G, Dv] — k itself when v is
+    None — to v_cache [n_blocks, G, block, Dv], at slot_mapping."""
     T, G, D = k.shape
     bs = k_cache.shape[2]
     qf, kf = q.float(), k.float()
@@ -609,7 +609,7 @@ def qk_norm_rope_store(q: torch.Tensor, k: torch.Tensor, q_norm: torch.Tensor,
     slot = slot_mapping.long()
     blk, off = slot // bs, slot % bs
     k_cache[blk, :, off] = kn.to(k_cache.dtype)
-    v_cache[blk, :, off] = k.to(v_cache.dtype)
+    v_cache[blk, :, off] = (k if v is None else v).to(v_cache.dtype)
 
 
 def sink_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -661,9 +661,10 @@ def sink_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
 def short_conv(x: torch.Tensor, w: torch.Tensor, state: torch.Tensor,
                state_slots: torch.Tensor, cu_seqlens: torch.Tensor,
                seq_idx: torch.Tensor, positions: torch.Tensor,
-               silu: bool = True) -> torch.Tensor:
-    """Causal per-channel conv over time (+ silu) -> fp32 [T, C]. x [T, C]
-    may be a strided column slice; w [taps, C] tap-major (last row is the
+               silu: bool = True, bias: Optional[torch.Tensor] = None,
+               out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
+    """Causal per-channel conv over time (+ bias [C]) (+ silu) -> out_dtype
+    [T, C]. x [T, C] may be a strided column slice; w [taps, C] tap-major (last row is the
     current token's); state [n_slots, taps-1, C] holds each sequence's last
     taps-1 inputs and is advanced in place. Rows before position 0 are zero
     by select."""
@@ -671,6 +672,8 @@ def short_conv(x: torch.Tensor, w: torch.Tensor, state: torch.Tensor,
     K = w.shape[0] - 1
     wf, xf = w.float(), x.float()
     out = xf * wf[K]
+    if bias is not None:
+        out = out + bias.float()
     if K > 0:
         sidx = seq_idx.long()
         rows = torch.arange(T, device=x.device)
@@ -697,7 +700,7 @@ def short_conv(x: torch.Tensor, w: torch.Tensor, state: torch.Tensor,
         state[st[live]] = new[live]
     if silu:
         out = torch.nn.functional.silu(out)
-    return out
+    return out.to(out_dtype)
 
 
 def delta_gates(qk: torch.Tensor, n_qk_heads: int, dim: int, b: torch.Tensor,
@@ -1122,15 +1125,16 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
              softcap: float, talk: Optional[torch.Tensor],
              sink: Optional[torch.Tensor],
              head_gate: Optional[torch.Tensor], window: int,
-             out: torch.Tensor,
-             dist: Optional[torch.Tensor] = None) -> None:
+             out: torch.Tensor, dist: Optional[torch.Tensor] = None,
+             out_scale: float = 1.0, keep_first: int = 0) -> None:
     """Grouped-query attention over the pages. Scores q . k (the score
     scale is already in q); dist fp32 [2, H] = (a, b): s_h <- s_h -
     a_h ln(1 + b_h d), d the distance between row and key; softcap > 0: s <- softcap tanh(s / softcap);
     talk fp32 [H, H]: s_h <- sum_g talk[h, g] s_g at every (row, key),
     BEFORE the softmax. Row t at position p of chunk b sees cached positions
-    j <= p (j > p - window when window > 0). sink fp32 [H]: exp(sink_h)
-    joins the denominator without a value. head_gate [T, H] raw (strided
+    j <= p (when window > 0 only j > p - window or j < keep_first). sink
+    fp32 [H]: exp(sink_h) joins the denominator without a value. out_scale
+    multiplies the result. head_gate [T, H] raw (strided
     view): head h's output times sigmoid(head_gate[t, h]).
     out [T, H * Dv] (strided view)."""
     T, H, D = q.shape
@@ -1145,7 +1149,8 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         pos = positions[lo:hi].long()
         k_lo = max(0, int(pos.min()) - window + 1) if window > 0 else 0
         k_hi = int(pos.max()) + 1
-        kpos = torch.arange(k_lo, k_hi, device=q.device)
+        kpos = torch.cat([torch.arange(min(keep_first, k_lo)),
+                          torch.arange(k_lo, k_hi)]).to(q.device)
         blk = block_table[b].long()[kpos // bs]
         keys = k_cache[blk, :, kpos % bs].float()          # [S, G, D]
         vals = v_cache[blk, :, kpos % bs].float()          # [S, G, Dv]
@@ -1161,7 +1166,7 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
             s = torch.einsum("hg,gts->hts", talk.float(), s)
         dead = d < 0
         if window > 0:
-            dead = dead | (d >= window)
+            dead = dead | ((d >= window) & (kpos >= keep_first)[None])
         s = s.masked_fill(dead[None], float("-inf"))
         m = s.max(-1, keepdim=True).values
         if sink is not None:
@@ -1176,7 +1181,7 @@ def gqa_attn(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
         res[lo:hi] = o.reshape(hi - lo, H, Dv)
     if head_gate is not None:
         res = res * torch.sigmoid(head_gate.float())[..., None]
-    out.copy_(res.view(T, H * Dv).to(out.dtype))
+    out.copy_((res.view(T, H * Dv) * out_scale).to(out.dtype))
 
 
 def min_gru(z: torch.Tensor, x: torch.Tensor, g: torch.Tensor,
@@ -1303,8 +1308,152 @@ def proj_norm_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
     v_cache[blk, :, off] = vn.to(v_cache.dtype)
 
 
+# --------------------------------------------- scaled parallel-form stacks
+#
+# Mechanisms of stacks whose layers are x += s1 * mixer(n1(x)) + s2 *
+# ffn(n2(x)) with vectors s1, s2 and two weighted norms of the same x,
+# followed by a per-token side input: sinusoidal position vectors, the fused
+# residual kernels, the side gate, the state-space recurrence and its gated
+# grouped norm.
+
+
+def sinusoid_freqs(width: int, device) -> torch.Tensor:
+    """float64 [ceil(width / 2)]: 10000^(-2i / width)."""
+    i = torch.arange((width + 1) // 2, dtype=torch.float64)
+    return torch.pow(torch.tensor(10000.0, dtype=torch.float64),
+                     -2.0 * i / width).to(device)
+
+
+def embed_sinusoid(ids: torch.Tensor, table: torch.Tensor, scale: float,
+                   positions: torch.Tensor, freqs: torch.Tensor
+                   ) -> torch.Tensor:
+    """fp32 [T, W]: table[id] * scale, plus sin(p f_i) at column 2i and
+    cos(p f_i) at column 2i + 1 (float64 angles, rounded once)."""
+    W = table.shape[1]
+    ang = positions.double()[:, None] * freqs
+    pe = torch.stack([ang.sin(), ang.cos()], dim=-1).flatten(1)[:, :W]
+    return table[ids.long()].float() * scale + pe.float()
+
+
+def add_norm_pair(resid: torch.Tensor, y: Optional[torch.Tensor],
+                  w_post: Optional[torch.Tensor], wa: Optional[torch.Tensor],
+                  wb: Optional[torch.Tensor], eps: float,
+                  out_dtype: torch.dtype):
+    """resid (fp32, in place) += unit(y) * w_post when y is given; returns
+    (unit(resid) * wa, unit(resid) * wb), None where the weight is None."""
+    if y is not None:
+        resid.add_(rmsnorm_f32(y, w_post, eps, torch.float32))
+    return tuple(None if w is None else rmsnorm_f32(resid, w, eps, out_dtype)
+                 for w in (wa, wb))
+
+
+def scaled_add(resid: torch.Tensor, y1: torch.Tensor, s1: torch.Tensor,
+               y2: Optional[torch.Tensor], s2: Optional[torch.Tensor],
+               y3: Optional[torch.Tensor], out_dtype: torch.dtype
+               ) -> torch.Tensor:
+    """resid (fp32, in place) += s1 * y1 [+ s2 * (y2 [+ y3])]; s1, s2 fp32
+    [W]. Returns resid in out_dtype (resid itself when that is fp32)."""
+    add = y1.float() * s1
+    if y2 is not None:
+        t = y2.float()
+        if y3 is not None:
+            t = t + y3.float()
+        add = add + t * s2
+    resid.add_(add)
+    return resid.to(out_dtype)
+
+
+def side_gate(g: torch.Tensor, table: torch.Tensor, offset: int,
+              ids: torch.Tensor) -> torch.Tensor:
+    """g [T, d] -> gelu_tanh(g) * table[ids, offset : offset + d]."""
+    e = table[ids.long(), offset : offset + g.shape[1]].float()
+    gf = torch.nn.functional.gelu(g.float(), approximate="tanh")
+    return (gf * e).to(g.dtype)
+
+
+SSD_CHUNK = 64
+
+
+def ssd_scan(xbc: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor,
+             rate: torch.Tensor, skip: torch.Tensor, groups: int,
+             state: torch.Tensor, state_slots: torch.Tensor,
+             cu_seqlens: torch.Tensor, positions: torch.Tensor
+             ) -> torch.Tensor:
+    """State-space recurrence, fp32. xbc [T, H*V + 2*G*N] holds x | B | C
+    (after their convolution), dt [T, H] the raw step sizes (strided views);
+    head h reads group h // (H/G). Per token and head, with
+    d = softplus(dt + dt_bias): S <- exp(-rate d) S + d B x^T;
+    y = S^T C + skip x. state [n_slots, H, N, V] fp32 is read unless the
+    chunk starts at position 0 and advanced in place. Evaluated in pieces:
+    inside one, exp of summed log decays weights C B^T; the carried state
+    enters with its own decay. Returns y fp32 [T, H*V]."""
+    H, N, V = state.shape[1:]
+    G, T = groups, xbc.shape[0]
+    f = xbc.float()
+    x = f[:, : H * V].view(T, H, V)
+    own = torch.arange(H, device=xbc.device) // (H // G)
+    Bm = f[:, H * V : H * V + G * N].view(T, G, N)[:, own]
+    Cm = f[:, H * V + G * N :].view(T, G, N)[:, own]
+    d = torch.nn.functional.softplus(dt.float() + dt_bias, threshold=30.0)
+    la = -rate * d                                          # log decay [T, H]
+    out = torch.empty(T, H, V, dtype=torch.float32, device=xbc.device)
+    cu = cu_seqlens.tolist()
+    for b in range(len(cu) - 1):
+        lo, hi = cu[b], cu[b + 1]
+        if hi == lo:
+            continue
+        slot = int(state_slots[b])
+        if int(positions[lo]) == 0:
+            S = torch.zeros(H, N, V, dtype=torch.float32, device=xbc.device)
+        else:
+            S = state[slot].clone()
+        for c0 in range(lo, hi, SSD_CHUNK):
+            c1 = min(hi, c0 + SSD_CHUNK)
+            A = la[c0:c1].cumsum(0).t()                     # [H, n]
+            xc = x[c0:c1].transpose(0, 1)                   # [H, n, V]
+            bc, cc = Bm[c0:c1].transpose(0, 1), Cm[c0:c1].transpose(0, 1)
+            dc = d[c0:c1].t()
+            L = torch.exp((A[:, :, None] - A[:, None, :]).clamp(max=0.0))
+            L = torch.tril(L) * dc[:, None, :]
+            o = torch.bmm(torch.bmm(cc, bc.transpose(1, 2).contiguous()) * L,
+                          xc)
+            o = o + torch.bmm(cc, S) * torch.exp(A)[..., None]
+            out[c0:c1] = (o + skip[:, None, None] * xc).transpose(0, 1)
+            tail = torch.exp(A[:, -1:] - A) * dc            # [H, n]
+            S = S * torch.exp(A[:, -1])[:, None, None] + torch.bmm(
+                (bc * tail[..., None]).transpose(1, 2).contiguous(), xc)
+        state[slot] = S
+    return out.view(T, H * V)
+
+
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, w: torch.Tensor,
+                     groups: int, eps: float, out: torch.Tensor,
+                     out_scale: float) -> None:
+    """out [T, N] (strided view) <- group_norm(y * silu(z)) * w * out_scale:
+    the gate first, then each of `groups` equal consecutive parts divided by
+    its own root mean square. y fp32 [T, N], z [T, N] raw (strided view)."""
+    v = y * torch.nn.functional.silu(z.float())
+    out.copy_((group_rmsnorm(v, w, groups, eps, torch.float32) *
+               out_scale).to(out.dtype))
+
 
 # ------------------------------------------------------- routed experts
+
+
+def routed_relu2(z: torch.Tensor, weights: torch.Tensor, idx: torch.Tensor,
+                 n_experts: int, ff: int) -> torch.Tensor:
+    """z [T, E*ff + n] (input products of every expert, then n columns that
+    every token uses) -> same shape: relu(w z)^2 with the token's weight for
+    the expert (zero where idx [T, k] does not name it); relu(z)^2 in the
+    last n columns."""
+    T = z.shape[0]
+    full = torch.zeros(T, n_experts, dtype=torch.float32, device=z.device)
+    full.scatter_(1, idx.long(), weights)
+    a = torch.relu(z.float())
+    r = a[:, : n_experts * ff].view(T, n_experts, ff) * full[..., None]
+    r = torch.where((full != 0)[..., None], r, torch.zeros_like(r))
+    y = torch.cat([r.reshape(T, -1), a[:, n_experts * ff :]], dim=1)
+    return (y * y).to(z.dtype)
 
 
 def routed_silu_glu(gu: torch.Tensor, weights: torch.Tensor,
