@@ -143,7 +143,8 @@ __global__ __launch_bounds__(64) void attn_prefill_basic(
 // first window are skipped. head_gate (optional, bf16 [tokens, nq] with row
 // stride s_g): head h's output times sigmoid(head_gate[t, h]). DIST:
 // dist [2, nq] = (a, b), a_h ln(1 + b_h d) is taken off a score whose key
-// lies d positions back.
+// lies d positions back. KEEP: with a window, the first `keep` positions stay
+// visible to every later row (their tiles are visited first).
 //
 // MODE 1 / MODE 2 split the kernel around a score buffer, for attention
 // whose scores are mixed across heads before the softmax: MODE 1 stops
@@ -156,7 +157,7 @@ __global__ __launch_bounds__(64) void attn_prefill_basic(
 // a row is key kv_lo + col, kv_lo being the first key the row's 64-query
 // tile visits. blockIdx.x counts tiles from qt0.
 template <int HD, bool PAGED, typename KVT, bool HILO = false, int MODE = 0,
-          bool DIST = false>
+          bool DIST = false, bool KEEP = false>
 __global__ __launch_bounds__(256) void attn_prefill_mfma(
     const unsigned short* __restrict__ q,
     const KVT* __restrict__ k,  // PAGED: k_cache [nb,nkv,bs,hd]
@@ -170,7 +171,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
     int window = 0, const unsigned short* __restrict__ head_gate = nullptr,
     long s_g = 0, float* __restrict__ score_buf = nullptr, int qt0 = 0,
     int qt_rows = 0, long ctx = 0, float softcap = 0.f,
-    const float* __restrict__ dist = nullptr) {
+    const float* __restrict__ dist = nullptr, int keep = 0) {
     constexpr int KSTEPS = HD / 32;
     const int seq = blockIdx.z;
     const int h = blockIdx.y;
@@ -240,7 +241,9 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
     const int kv_lo =
         window > 0 ? max(0, hist + q0 - window + 1) / PF_TN * PF_TN : 0;
 
-    for (int kb = kv_lo; kb < kv_end; kb += PF_TN) {
+    for (int kb = KEEP ? 0 : kv_lo; kb < kv_end; kb += PF_TN) {
+        // past the kept keys' tiles: on to the window
+        if (KEEP && kb >= keep && kb < kv_lo) kb = kv_lo;
         // ---- stage K tile [32][HD] and V^T tile [HD][32]
         __syncthreads();
         {
@@ -341,7 +344,8 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
                     sfrag[f][r] -= da * __logf(1.f + db * d);
                 }
                 if (key > hist + qrow || qrow >= QL || key >= kv_end ||
-                    (window > 0 && key <= hist + qrow - window))
+                    (window > 0 && key <= hist + qrow - window &&
+                     !(KEEP && key < keep)))
                     sfrag[f][r] = -1e30f;
                 pmax[r] = fmaxf(pmax[r], sfrag[f][r]);
             }
@@ -530,29 +534,32 @@ extern "C" void launch_attn_prefill_paged(
 // scale and a strided output (a column slice of a wider buffer). bf16,
 // head size 64 or 128 (returns nonzero otherwise); scale is applied by the
 // caller (folded into q). window 0: causal without a window; head_gate and
-// dist optional (see the kernel).
+// dist optional, keep > 0 not together with dist (see the kernel).
 extern "C" int launch_attn_prefill_paged_sink(
     const unsigned short* q, long s_q, const unsigned short* k_cache,
     const unsigned short* v_cache, const int* cu, const int* block_table,
     const int* seq_lens, unsigned short* out, long s_o, int nseq, int nq,
     int nkv, int hd, int W, int bs, int max_qlen, const float* sink,
     float out_scale, int window, const unsigned short* head_gate, long s_g,
-    const float* dist, hipStream_t stream) {
+    const float* dist, int keep, hipStream_t stream) {
+    if (keep > 0 && dist) return 1;
     if (hd != 64 && hd != 128) return 1;
     if (nseq == 0 || max_qlen == 0) return 0;
     const int tiles = (max_qlen + PF_TM - 1) / PF_TM;
     dim3 grid(tiles, nq, nseq);
     const int smem = prefill_mfma_smem(hd, 1);
-#define PS_LAUNCH(HDV, DI)                                                    \
+#define PS_LAUNCH(HDV, DI, KP)                                                \
     hipLaunchKernelGGL(                                                       \
-        (attn_prefill_mfma<HDV, true, unsigned short, true, 0, DI>), grid,    \
-        dim3(256), smem, stream, q, k_cache, v_cache, cu, block_table,        \
+        (attn_prefill_mfma<HDV, true, unsigned short, true, 0, DI, KP>),      \
+        grid, dim3(256), smem, stream, q, k_cache, v_cache, cu, block_table,  \
         seq_lens, out, nq, nkv, s_q, 0, 0, W, bs, 1.f, sink, out_scale, s_o,  \
-        window, head_gate, s_g, nullptr, 0, 0, 0, 0.f, dist)
-    if (hd == 128 && dist) PS_LAUNCH(128, true);
-    else if (hd == 128) PS_LAUNCH(128, false);
-    else if (dist) PS_LAUNCH(64, true);
-    else PS_LAUNCH(64, false);
+        window, head_gate, s_g, nullptr, 0, 0, 0, 0.f, dist, keep)
+    if (hd == 128 && keep > 0) PS_LAUNCH(128, false, true);
+    else if (keep > 0) PS_LAUNCH(64, false, true);
+    else if (hd == 128 && dist) PS_LAUNCH(128, true, false);
+    else if (hd == 128) PS_LAUNCH(128, false, false);
+    else if (dist) PS_LAUNCH(64, true, false);
+    else PS_LAUNCH(64, false, false);
 #undef PS_LAUNCH
     return 0;
 }

@@ -404,6 +404,7 @@ void register_sandwich_ops(pybind11::module_& m);  // sandwich_ext.cpp
 void register_gated_ops(pybind11::module_& m);  // gated_ext.cpp
 void register_tanh_ops(pybind11::module_& m);  // tanh_ext.cpp
 void register_moe_ops(pybind11::module_& m);  // moe_ext.cpp
+void register_scaled_ops(pybind11::module_& m);  // scaled_ext.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     register_hybrid_ops(m);
@@ -411,6 +412,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
     register_gated_ops(m);
     register_tanh_ops(m);
     register_moe_ops(m);
+    register_scaled_ops(m);
     m.def("rmsnorm", &rmsnorm, "fused RMSNorm (bf16)");
     m.def("fused_add_rmsnorm", &fused_add_rmsnorm,
           "residual += x; y = rmsnorm(residual)");

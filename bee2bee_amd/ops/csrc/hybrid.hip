@@ -195,8 +195,8 @@ __global__ void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ y,
 }
 
 // ------------------------------------------------------- input convolution
-// out[t] = [h[t] +] sum_d w[K-d][c] * h[t-d], d = 0..K (K = taps-1), then
-// silu when SILU. RES adds the input itself (the whole-width conv of the
+// out[t] = [h[t] +] sum_d w[K-d][c] * h[t-d] [+ bias[c]], d = 0..K
+// (K = taps-1), then silu when SILU. RES adds the input itself (the whole-width conv of the
 // sandwich layers); the short conv of a delta mixer is plain and activated.
 // h may be a column slice of a wider buffer (row stride hs); out is
 // contiguous [T, C] of type OT. Rows before the chunk come from the
@@ -209,7 +209,8 @@ __global__ void canon_conv_kernel(const T* __restrict__ h, long hs,
                                   const int* __restrict__ cu,
                                   const int* __restrict__ seq_idx,
                                   const int* __restrict__ positions,
-                                  OT* __restrict__ out, int C, int K) {
+                                  OT* __restrict__ out, int C, int K,
+                                  const float* __restrict__ bias) {
     const long t = blockIdx.x;
     const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
     if (c >= C) return;
@@ -233,6 +234,11 @@ __global__ void canon_conv_kernel(const T* __restrict__ h, long hs,
         ldv<float, VEC>(w + (long)(K - d) * C + c, wv);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * v[j];
+    }
+    if (bias) {
+        ldv<float, VEC>(bias + c, wv);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) acc[j] += wv[j];
     }
     if (SILU) {
 #pragma unroll
@@ -454,8 +460,8 @@ __global__ void delta_gates_kernel(float* __restrict__ qk, long qs, int NQ,
 // ------------------------------------- query/key norm, rotation, page store
 // Workgroup per token, a wave per head in turn (H query heads, then G key
 // heads). Query head: q <- rotate(unit(q) * wq) * q_mult[h] in place. Key
-// head: rotate(unit(k) * wk) -> k_cache, k as projected -> v_cache (pages
-// [n_blocks, G, bs, D]). Rotation pairs dim i with i + dims/2 over the
+// head: rotate(unit(k) * wk) -> k_cache; v, or k as projected when v is null
+// (Dv = D), -> v_cache (pages [n_blocks, G, bs, D | Dv]). Rotation pairs dim i with i + dims/2 over the
 // first `dims` coordinates; cos/sin fp32 tables [max_pos, dims/2].
 constexpr int QKN_MAXD = 512;
 template <typename T>
@@ -469,7 +475,8 @@ qk_norm_rope_store_kernel(T* __restrict__ q, long q_tok, int H,
                           const float* __restrict__ sin_t,
                           const float* __restrict__ q_mult,
                           T* __restrict__ k_cache, T* __restrict__ v_cache,
-                          int bs, const int* __restrict__ slot_mapping) {
+                          int bs, const int* __restrict__ slot_mapping,
+                          const T* __restrict__ v, long v_tok, int Dv) {
     __shared__ float buf[4][QKN_MAXD];
     const long t = blockIdx.x;
     const int wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
@@ -494,7 +501,12 @@ qk_norm_rope_store_kernel(T* __restrict__ q, long q_tok, int H,
         const float mul = is_q ? q_mult[hh] : 1.f;
         T* dst = is_q ? q + t * q_tok + (long)hh * D
                       : k_cache + ((blk * G + g) * bs + off) * D;
-        T* vdst = is_q ? nullptr : v_cache + ((blk * G + g) * bs + off) * D;
+        T* vdst = is_q ? nullptr : v_cache + ((blk * G + g) * bs + off) * Dv;
+        if (vdst && v) {
+            const T* vsrc = v + t * v_tok + (long)g * Dv;
+            for (int i = lane; i < Dv; i += WAVE) vdst[i] = vsrc[i];
+            vdst = nullptr;
+        }
         // every lane has written its nb entries before any lane reads a
         // partner's: the wave_sum above is a full-wave exchange, and the
         // LDS writes of a wave complete in order before its later reads
@@ -627,7 +639,7 @@ static void conv_dispatch(const void* h, long hs, const float* w, void* state,
                           const int* state_slots, const int* cu,
                           const int* seq_idx, const int* positions, void* out,
                           long T_, int B, int C, int K, bool vec4,
-                          hipStream_t s) {
+                          const float* bias, hipStream_t s) {
     const int th = C >= 256 ? 256 : 64;
     const int vec = vec4 ? 4 : 1;
     const int lanes = (C + vec - 1) / vec;
@@ -635,11 +647,11 @@ static void conv_dispatch(const void* h, long hs, const float* w, void* state,
     if (vec4)
         canon_conv_kernel<T, OT, 4, RES, SILU><<<g1, th, 0, s>>>(
             (const T*)h, hs, w, (const T*)state, state_slots, cu, seq_idx,
-            positions, (OT*)out, C, K);
+            positions, (OT*)out, C, K, bias);
     else
         canon_conv_kernel<T, OT, 1, RES, SILU><<<g1, th, 0, s>>>(
             (const T*)h, hs, w, (const T*)state, state_slots, cu, seq_idx,
-            positions, (OT*)out, C, K);
+            positions, (OT*)out, C, K, bias);
     if (K > 0)
         canon_state_kernel<T><<<g2, th, 0, s>>>(
             (const T*)h, hs, (T*)state, state_slots, cu, C, K);
@@ -656,28 +668,33 @@ extern "C" void launch_canon_conv(const void* h, const float* w, void* state,
     if (f32)
         conv_dispatch<float, float, true, false>(
             h, C, w, state, state_slots, cu, seq_idx, positions, out, T, B, C,
-            K, v4, s);
+            K, v4, nullptr, s);
     else
         conv_dispatch<unsigned short, unsigned short, true, false>(
             h, C, w, state, state_slots, cu, seq_idx, positions, out, T, B, C,
-            K, v4, s);
+            K, v4, nullptr, s);
 }
 
-// conv(h) [silu] -> fp32, h a column slice with row stride hs
+// conv(h) [+ bias] [silu] -> fp32, or bf16 from bf16 (out_f32 0); h a column
+// slice with row stride hs
 extern "C" void launch_short_conv(const void* h, long hs, const float* w,
                                   void* state, const int* state_slots,
                                   const int* cu, const int* seq_idx,
-                                  const int* positions, float* out, long T,
+                                  const int* positions, void* out, long T,
                                   int B, int C, int K, int silu, int vec4,
-                                  int f32, hipStream_t s) {
+                                  int f32, const float* bias, int out_f32,
+                                  hipStream_t s) {
     if (T == 0) return;
-#define SC_CALL(TT, SI)                                                       \
-    conv_dispatch<TT, float, false, SI>(h, hs, w, state, state_slots, cu,     \
-                                        seq_idx, positions, out, T, B, C, K,  \
-                                        vec4 != 0, s)
-    if (f32) { if (silu) SC_CALL(float, true); else SC_CALL(float, false); }
-    else if (silu) SC_CALL(unsigned short, true);
-    else SC_CALL(unsigned short, false);
+#define SC_CALL(TT, OT, SI)                                                   \
+    conv_dispatch<TT, OT, false, SI>(h, hs, w, state, state_slots, cu,        \
+                                     seq_idx, positions, out, T, B, C, K,     \
+                                     vec4 != 0, bias, s)
+    if (f32 && silu) SC_CALL(float, float, true);
+    else if (f32) SC_CALL(float, float, false);
+    else if (out_f32 && silu) SC_CALL(unsigned short, float, true);
+    else if (out_f32) SC_CALL(unsigned short, float, false);
+    else if (silu) SC_CALL(unsigned short, unsigned short, true);
+    else SC_CALL(unsigned short, unsigned short, false);
 #undef SC_CALL
 }
 
@@ -762,20 +779,21 @@ extern "C" int launch_qk_norm_rope_store(
     const float* wq, const float* wk, float eps, int dims,
     const int* positions, const float* cos_t, const float* sin_t,
     const float* q_mult, void* k_cache, void* v_cache, int bs,
-    const int* slot_mapping, long T, int f32, hipStream_t s) {
+    const int* slot_mapping, const void* v, long v_tok, int Dv, long T,
+    int f32, hipStream_t s) {
     if (D > QKN_MAXD) return 1;
     if (T == 0) return 0;
     if (f32)
         qk_norm_rope_store_kernel<float><<<T, 256, 0, s>>>(
             (float*)q, q_tok, H, (const float*)k, k_tok, G, D, wq, wk, eps,
             dims, positions, cos_t, sin_t, q_mult, (float*)k_cache,
-            (float*)v_cache, bs, slot_mapping);
+            (float*)v_cache, bs, slot_mapping, (const float*)v, v_tok, Dv);
     else
         qk_norm_rope_store_kernel<unsigned short><<<T, 256, 0, s>>>(
             (unsigned short*)q, q_tok, H, (const unsigned short*)k, k_tok, G,
             D, wq, wk, eps, dims, positions, cos_t, sin_t, q_mult,
             (unsigned short*)k_cache, (unsigned short*)v_cache, bs,
-            slot_mapping);
+            slot_mapping, (const unsigned short*)v, v_tok, Dv);
     return 0;
 }
 

@@ -45,8 +45,9 @@ int launch_lightning(const void*, const void*, const void*, long,
                      float*, float*, int, int, int, int, int, int, int,
                      const float*, const float*, int, float, hipStream_t);
 void launch_short_conv(const void*, long, const float*, void*, const int*,
-                       const int*, const int*, const int*, float*, long, int,
-                       int, int, int, int, int, hipStream_t);
+                       const int*, const int*, const int*, void*, long, int,
+                       int, int, int, int, int, const float*, int,
+                       hipStream_t);
 void launch_add_rmsnorm_w(float*, const void*, const float*, void*, long, int,
                           float, int, int, hipStream_t);
 void launch_relu2(const void*, long, void*, long, long, int, int, int,
@@ -61,7 +62,7 @@ int launch_qk_norm_rope_store(void*, long, int, const void*, long, int, int,
                               const float*, const float*, float, int,
                               const int*, const float*, const float*,
                               const float*, void*, void*, int, const int*,
-                              long, int, hipStream_t);
+                              const void*, long, int, long, int, hipStream_t);
 int launch_delta_rule(const float*, const float*, long, const float*, long,
                       const float*, const float*, int, float*, const int*,
                       const int*, const int*, float*, int, int, int, int, int,
@@ -73,11 +74,11 @@ int launch_attn_prefill_paged_sink(const unsigned short*, long,
                                    long, int, int, int, int, int, int, int,
                                    const float*, float, int,
                                    const unsigned short*, long, const float*,
-                                   hipStream_t);
+                                   int, hipStream_t);
 int launch_sink_attn(const void*, long, const void*, const void*, const int*,
                      int, const int*, const int*, const float*, void*, long,
                      float, float*, float*, int, int, int, int, int, int, int,
-                     int, int, const void*, long, const float*,
+                     int, int, const void*, long, const float*, int,
                      hipStream_t);
 }
 
@@ -491,7 +492,9 @@ void relu2(const Tensor& x, Tensor& out) {
 
 Tensor short_conv(const Tensor& x, const Tensor& w, Tensor& state,
                   const Tensor& state_slots, const Tensor& cu,
-                  const Tensor& seq_idx, const Tensor& positions, bool silu) {
+                  const Tensor& seq_idx, const Tensor& positions, bool silu,
+                  const std::optional<Tensor>& bias,
+                  at::ScalarType out_dtype) {
     const int c = act_code(x, "x");
     check_f32(w, "w");
     check_i32(state_slots, "state_slots");
@@ -512,14 +515,22 @@ Tensor short_conv(const Tensor& x, const Tensor& w, Tensor& state,
                     state.scalar_type() == x.scalar_type() &&
                     state.dim() == 3 && state.size(1) == K &&
                     state.size(2) == C);
-    Tensor out = torch::empty({T, (long)C},
-                              x.options().dtype(torch::kFloat32));
+    TORCH_CHECK(out_dtype == torch::kFloat32 || out_dtype == x.scalar_type(),
+                "short_conv: output is fp32 or the input's type");
+    const float* bp = nullptr;
+    if (bias.has_value()) {
+        check_f32(*bias, "bias");
+        TORCH_CHECK(bias->numel() == C);
+        bp = bias->data_ptr<float>();
+    }
+    Tensor out = torch::empty({T, (long)C}, x.options().dtype(out_dtype));
     launch_short_conv(x.data_ptr(), x.stride(0), w.data_ptr<float>(),
                       K > 0 ? state.data_ptr() : nullptr,
                       state_slots.data_ptr<int>(), cu.data_ptr<int>(),
                       seq_idx.data_ptr<int>(), positions.data_ptr<int>(),
-                      out.data_ptr<float>(), T, B, C, K, silu ? 1 : 0,
-                      aligned4(x) ? 1 : 0, c, stream());
+                      out.data_ptr(), T, B, C, K, silu ? 1 : 0,
+                      aligned4(x) ? 1 : 0, c, bp,
+                      out_dtype == torch::kFloat32 ? 1 : 0, stream());
     return out;
 }
 
@@ -618,7 +629,8 @@ void qk_norm_rope_store(Tensor& q, const Tensor& k, const Tensor& q_norm,
                         const std::optional<Tensor>& cos_t,
                         const std::optional<Tensor>& sin_t,
                         const Tensor& q_mult, Tensor& k_cache,
-                        Tensor& v_cache, const Tensor& slot_mapping) {
+                        Tensor& v_cache, const Tensor& slot_mapping,
+                        const std::optional<Tensor>& v) {
     const int c = act_code(q, "q");
     check_f32(q_norm, "q_norm");
     check_f32(k_norm, "k_norm");
@@ -645,17 +657,32 @@ void qk_norm_rope_store(Tensor& q, const Tensor& k, const Tensor& q_norm,
         cp = cos_t->data_ptr<float>();
         sp = sin_t->data_ptr<float>();
     }
+    int Dv = D;
+    const void* vp = nullptr;
+    long v_tok = 0;
+    if (v.has_value()) {
+        TORCH_CHECK(v->is_cuda() && v->dim() == 3 && v->size(0) == T &&
+                    v->size(1) == G && v->stride(2) == 1 &&
+                    v->stride(1) == v->size(2) &&
+                    v->scalar_type() == q.scalar_type());
+        Dv = (int)v->size(2);
+        vp = v->data_ptr();
+        v_tok = v->stride(0);
+    }
     for (const Tensor* t : {&k_cache, &v_cache})
         TORCH_CHECK(t->is_cuda() && t->scalar_type() == q.scalar_type() &&
                     t->is_contiguous() && t->dim() == 4 && t->size(1) == G &&
-                    t->size(3) == D && t->sizes() == k_cache.sizes());
+                    t->size(0) == k_cache.size(0) &&
+                    t->size(2) == k_cache.size(2));
+    TORCH_CHECK(k_cache.size(3) == D && v_cache.size(3) == Dv);
     TORCH_CHECK(positions.numel() == T && slot_mapping.numel() == T);
     const int rc = launch_qk_norm_rope_store(
         q.data_ptr(), q.stride(0), H, k.data_ptr(), k.stride(0), G, D,
         q_norm.data_ptr<float>(), k_norm.data_ptr<float>(), (float)eps,
         (int)rope_dims, positions.data_ptr<int>(), cp, sp,
         q_mult.data_ptr<float>(), k_cache.data_ptr(), v_cache.data_ptr(),
-        (int)k_cache.size(2), slot_mapping.data_ptr<int>(), T, c, stream());
+        (int)k_cache.size(2), slot_mapping.data_ptr<int>(), vp, v_tok, Dv, T,
+        c, stream());
     TORCH_CHECK(rc == 0, "qk_norm_rope_store: head dim must be <= 512");
 }
 
@@ -665,7 +692,7 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
                const std::optional<Tensor>& sink, int64_t window, Tensor& out,
                double out_scale, int64_t max_qlen,
                const std::optional<Tensor>& head_gate,
-               const std::optional<Tensor>& dist) {
+               const std::optional<Tensor>& dist, int64_t keep_first) {
     const int c = act_code(q, "q");
     check_i32(block_table, "block_table");
     check_i32(positions, "positions");
@@ -681,7 +708,10 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
                 v_cache.size(1) == G && v_cache.size(2) == bs &&
                 v_cache.scalar_type() == q.scalar_type());
     const int Dv = (int)v_cache.size(3);
-    TORCH_CHECK(G >= 1 && H % G == 0 && window >= 0);
+    TORCH_CHECK(G >= 1 && H % G == 0 && window >= 0 && keep_first >= 0);
+    // without a window nothing is out of sight
+    const int keep = window > 0 ? (int)std::min<int64_t>(keep_first, 1 << 30)
+                                : 0;
     TORCH_CHECK(block_table.dim() == 2 && positions.numel() == Tn &&
                 seq_idx.numel() == Tn);
     check_slice(out, Tn, (long)H * Dv, q.scalar_type(), "out");
@@ -712,7 +742,8 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
     // pair, window-aware tile skipping, and the sink and head gate in its
     // epilogue); single rows in the same step ride along. fp32, other head
     // sizes and pure decode steps take the generic kernel below.
-    if (c == 0 && max_qlen >= 16 && D == Dv && (D == 64 || D == 128)) {
+    if (c == 0 && max_qlen >= 16 && D == Dv && (D == 64 || D == 128) &&
+        !(keep > 0 && dp)) {
         const long B = cu.numel() - 1;
         TORCH_CHECK(block_table.size(0) == B);
         Tensor last = cu.slice(0, 1, B + 1).to(torch::kLong) - 1;
@@ -727,14 +758,16 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
             (unsigned short*)out.data_ptr(), out.stride(0), (int)B, H, G, D,
             (int)block_table.size(1), bs, (int)max_qlen, sk,
             (float)out_scale, (int)window, (const unsigned short*)hg, hg_tok,
-            dp, stream());
+            dp, keep, stream());
         TORCH_CHECK(rc == 0, "sink_attn: matrix-core path refused a shape "
                              "its guard admitted");
         return;
     }
     // few rows (decode): split each row's keys over more waves, at least 64
     // keys per share of the longest context the tables can hold
-    const long ctx = window > 0 ? window : block_table.size(1) * (long)bs;
+    const long held = block_table.size(1) * (long)bs;
+    const long ctx = window > 0 ? std::min<long>(window + (long)keep, held)
+                                : held;
     // a wave serves up to 4 query heads of one key group (mixers.hip)
     const long group = H / G;
     const long units = H / (group % 4 == 0 ? 4 : group % 2 == 0 ? 2 : 1);
@@ -755,7 +788,7 @@ void sink_attn(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache,
         block_table.data_ptr<int>(), (int)block_table.size(1),
         positions.data_ptr<int>(), seq_idx.data_ptr<int>(), sk,
         out.data_ptr(), out.stride(0), (float)out_scale, pa, pm, (int)splits,
-        Tn, H, G, D, Dv, bs, (int)window, c, hg, hg_tok, dp, stream());
+        Tn, H, G, D, Dv, bs, (int)window, c, hg, hg_tok, dp, keep, stream());
     TORCH_CHECK(rc == 0, "sink_attn: head sizes must be <= 256");
 }
 
@@ -786,7 +819,12 @@ void register_hybrid_ops(pybind11::module_& m) {
           "resid(fp32) += y; out = unit(resid) * w");
     m.def("relu2", &relu2, "relu(x)^2 over column slices");
     m.def("short_conv", &short_conv,
-          "causal per-channel conv (+silu) with carried state -> fp32");
+          "causal per-channel conv (+bias, silu) with carried state",
+          pybind11::arg("x"), pybind11::arg("w"), pybind11::arg("state"),
+          pybind11::arg("state_slots"), pybind11::arg("cu_seqlens"),
+          pybind11::arg("seq_idx"), pybind11::arg("positions"),
+          pybind11::arg("silu"), pybind11::arg("bias") = std::nullopt,
+          pybind11::arg("out_dtype") = torch::kFloat32);
     m.def("delta_gates", &delta_gates,
           "unit q/k in place, beta and decay of a delta-rule step");
     m.def("delta_rule", &delta_rule,
@@ -794,7 +832,14 @@ void register_hybrid_ops(pybind11::module_& m) {
     m.def("head_gated_norm", &head_gated_norm,
           "per-head unit(o) * w * act(gate) into a column slice");
     m.def("qk_norm_rope_store", &qk_norm_rope_store,
-          "q/k head norm + rotation; keys and raw keys to the pages");
+          "q/k head norm + rotation; keys and values (or raw keys) to the "
+          "pages",
+          pybind11::arg("q"), pybind11::arg("k"), pybind11::arg("q_norm"),
+          pybind11::arg("k_norm"), pybind11::arg("eps"),
+          pybind11::arg("rope_dims"), pybind11::arg("positions"),
+          pybind11::arg("cos"), pybind11::arg("sin"), pybind11::arg("q_mult"),
+          pybind11::arg("k_cache"), pybind11::arg("v_cache"),
+          pybind11::arg("slot_mapping"), pybind11::arg("v") = std::nullopt);
     m.def("sink_attn", &sink_attn,
           "paged causal GQA softmax attention with a sink logit",
           pybind11::arg("q"), pybind11::arg("k_cache"),
@@ -804,5 +849,6 @@ void register_hybrid_ops(pybind11::module_& m) {
           pybind11::arg("window"), pybind11::arg("out"),
           pybind11::arg("out_scale"), pybind11::arg("max_qlen"),
           pybind11::arg("head_gate") = std::nullopt,
-          pybind11::arg("dist") = std::nullopt);
+          pybind11::arg("dist") = std::nullopt,
+          pybind11::arg("keep_first") = 0);
 }

@@ -869,7 +869,8 @@ delta_rule_kernel(const float* __restrict__ q, const float* __restrict__ k,
 // while the weights are read lane by lane. Scores, weights and accumulators are fp32; every score
 // multiplier is already in q. The softmax denominator also counts
 // exp(sink[h]) once when sink is given. Row t at position p sees cached
-// positions j <= p (j > p - window when window > 0). With gridDim.z > 1
+// positions j <= p (when window > 0 only j > p - window or j < keep: its
+// keys are numbered kept ones first, then the window's). With gridDim.z > 1
 // each split writes its (max, sum, partial) and sink_attn_combine merges.
 constexpr int SA_WAVES = 4;
 constexpr int SA_MAXD = 256;
@@ -1015,7 +1016,7 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
                  float* __restrict__ part_ml, int Tn, int H, int G, int D,
                  int Dv, int bs, int window,
                  const T* __restrict__ head_gate, long hg_tok,
-                 const float* __restrict__ dist) {
+                 const float* __restrict__ dist, int keep) {
     extern __shared__ __attribute__((aligned(16))) float sa_q[];
     const int wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
     const int t = blockIdx.x;
@@ -1026,11 +1027,13 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
     const int p = positions[t];
     const int g = h0 / (H / G);
     const int lo = window > 0 ? max(0, p - window + 1) : 0;
+    // visible keys by number: nkeep kept ones at 0.., then lo..p
+    const int nkeep = min(keep, lo), seen = nkeep + p + 1 - lo;
     // a split takes whole 64-key tiles, so no wave pays a full score pass
     // for a few keys; splits past the end stay empty (sum 0) for the merge
     const int per =
-        ((p + 1 - lo + nsplit - 1) / nsplit + WAVE - 1) / WAVE * WAVE;
-    const int klo = lo + split * per, khi = min(p + 1, klo + per);
+        ((seen + nsplit - 1) / nsplit + WAVE - 1) / WAVE * WAVE;
+    const int klo = split * per, khi = min(seen, klo + per);
     float* qv = sa_q + (long)wid * REP * D;
     for (int i = lane; i < REP * D; i += WAVE)
         qv[i] = ldf(q + (long)t * q_tok + (long)h0 * D + i);
@@ -1051,7 +1054,8 @@ sink_attn_kernel(const T* __restrict__ q, long q_tok,
         const bool valid = j < khi;
         // lanes past the end point at the share's last key: a row this
         // sequence wrote (their weights are 0, and 0 x garbage is not 0)
-        const int jc = min(j, khi - 1);
+        const int jn = min(j, khi - 1);
+        const int jc = jn < nkeep ? jn : jn - nkeep + lo;
         const int row = (bt[jc / bs] * G + g) * bs + jc % bs;
         float sc[REP], pj[REP];
 #pragma unroll
@@ -1418,7 +1422,7 @@ extern "C" int launch_delta_rule(const float* q, const float* k, long qk_tok,
         (const TT*)q, q_tok, (const TT*)k_cache, (const TT*)v_cache,          \
         block_table, bt_stride, positions, seq_idx, sink, (TT*)out, out_tok,  \
         out_scale, part_acc, part_ml, Tn, H, G, D, Dv, bs, window,            \
-        (const TT*)head_gate, hg_tok, dist)
+        (const TT*)head_gate, hg_tok, dist, keep)
 
 #define SA_CASE(N, P)                                                         \
     if (dpl == N && pair == P) {                                              \
@@ -1437,7 +1441,7 @@ static int sink_attn_dispatch(const void* q, long q_tok, const void* k_cache,
                               float* part_acc, float* part_ml, int splits,
                               int Tn, int H, int G, int D, int Dv, int bs,
                               int window, const void* head_gate, long hg_tok,
-                              const float* dist, hipStream_t s) {
+                              const float* dist, int keep, hipStream_t s) {
     // even value sizes: a lane owns coordinate pairs (one load for two)
     const bool pair = Dv % 2 == 0;
     int dpl = pair ? 2 * ((Dv + 2 * WAVE - 1) / (2 * WAVE))
@@ -1465,7 +1469,8 @@ static int sink_attn_dispatch(const void* q, long q_tok, const void* k_cache,
 // head_gate (optional, activation type, [Tn, H] with row stride hg_tok):
 // head h's output times sigmoid(head_gate[t, h]). dist (optional, fp32
 // [2, H] = (a, b)): a_h ln(1 + b_h d) is taken off a score whose key lies d
-// positions back. Returns nonzero when a head size exceeds 256.
+// positions back. keep: first positions that stay visible past the window.
+// Returns nonzero when a head size exceeds 256.
 extern "C" int launch_sink_attn(const void* q, long q_tok,
                                 const void* k_cache, const void* v_cache,
                                 const int* block_table, int bt_stride,
@@ -1475,18 +1480,18 @@ extern "C" int launch_sink_attn(const void* q, long q_tok,
                                 float* part_ml, int splits, int Tn, int H,
                                 int G, int D, int Dv, int bs, int window,
                                 int f32, const void* head_gate, long hg_tok,
-                                const float* dist, hipStream_t s) {
+                                const float* dist, int keep, hipStream_t s) {
     if (D > SA_MAXD || Dv > SA_MAXD) return 1;
     if (Tn == 0) return 0;
     if (f32)
         return sink_attn_dispatch<float>(
             q, q_tok, k_cache, v_cache, block_table, bt_stride, positions,
             seq_idx, sink, out, out_tok, out_scale, part_acc, part_ml, splits,
-            Tn, H, G, D, Dv, bs, window, head_gate, hg_tok, dist, s);
+            Tn, H, G, D, Dv, bs, window, head_gate, hg_tok, dist, keep, s);
     return sink_attn_dispatch<unsigned short>(
         q, q_tok, k_cache, v_cache, block_table, bt_stride, positions,
         seq_idx, sink, out, out_tok, out_scale, part_acc, part_ml, splits, Tn,
-        H, G, D, Dv, bs, window, head_gate, hg_tok, dist, s);
+        H, G, D, Dv, bs, window, head_gate, hg_tok, dist, keep, s);
 }
 
 // ---------------------------------------------------------------------------

@@ -168,6 +168,41 @@ routed_silu_glu_kernel(const T* __restrict__ gu, const float* __restrict__ wt,
     stn<T, VEC>(out + t * E * (long)I + c, y);
 }
 
+// --------------------------------------------- routed square of relu
+// z, out [T, E*I + n]: relu(w z)^2 in the columns of an expert the token
+// chose (w its routing weight, applied to what the expert reads), zeros,
+// without reading z, for the others; relu(z)^2 in the last n columns.
+template <typename T, int VEC>
+__global__ void __launch_bounds__(MO_THREADS)
+routed_relu2_kernel(const T* __restrict__ z, const float* __restrict__ wt,
+                    const int* __restrict__ idx, T* __restrict__ out, int E,
+                    int I, int N, int top_k) {
+    const int c = (blockIdx.y * MO_THREADS + threadIdx.x) * VEC;
+    if (c >= N) return;             // VEC = 4 only when 4 divides I and N
+    const long t = blockIdx.x;
+    const int e = c / I;
+    float w = e >= E ? 1.f : 0.f;
+    bool used = e >= E;
+    if (!used)
+        for (int j = 0; j < top_k; ++j)
+            if (idx[t * top_k + j] == e) {
+                w = wt[t * top_k + j];
+                used = true;
+            }
+    float y[VEC];
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) y[j] = 0.f;
+    if (used) {
+        ldn<T, VEC>(z + t * (long)N + c, y);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            const float r = fmaxf(w * y[j], 0.f);
+            y[j] = r * r;
+        }
+    }
+    stn<T, VEC>(out + t * (long)N + c, y);
+}
+
 }  // namespace
 
 // ---------------------------------------------------------------- launchers
@@ -213,4 +248,21 @@ extern "C" void launch_routed_silu_glu(const void* gu, const float* wt,
     else if (vec) RG_LAUNCH(unsigned short, 4);
     else RG_LAUNCH(unsigned short, 1);
 #undef RG_LAUNCH
+}
+
+extern "C" void launch_routed_relu2(const void* z, const float* wt,
+                                    const int* idx, void* out, long T, int E,
+                                    int I, int N, int top_k, int c, int vec,
+                                    hipStream_t s) {
+    if (T == 0) return;
+    const int per = MO_THREADS * (vec ? 4 : 1);
+    const dim3 grid((unsigned)T, (N + per - 1) / per);
+#define RR_LAUNCH(TT, V)                                                      \
+    routed_relu2_kernel<TT, V><<<grid, MO_THREADS, 0, s>>>(                   \
+        (const TT*)z, wt, idx, (TT*)out, E, I, N, top_k)
+    if (c && vec) RR_LAUNCH(float, 4);
+    else if (c) RR_LAUNCH(float, 1);
+    else if (vec) RR_LAUNCH(unsigned short, 4);
+    else RR_LAUNCH(unsigned short, 1);
+#undef RR_LAUNCH
 }

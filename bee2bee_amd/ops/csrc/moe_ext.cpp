@@ -17,6 +17,8 @@ void launch_moe_combine(const void*, const int*, const float*, void*, long,
                         int, int, int, int, hipStream_t);
 void launch_routed_silu_glu(const void*, const float*, const int*, void*, long,
                             int, int, int, int, int, hipStream_t);
+void launch_routed_relu2(const void*, const float*, const int*, void*, long,
+                         int, int, int, int, int, int, hipStream_t);
 }
 
 namespace {
@@ -104,6 +106,27 @@ Tensor routed_silu_glu(const Tensor& gu, const Tensor& weights,
     return out;
 }
 
+// z [T, E * ff + n]: the experts' input products, then n always-on columns
+Tensor routed_relu2(const Tensor& z, const Tensor& weights, const Tensor& idx,
+                    int64_t n_experts, int64_t ff) {
+    const int c = act_code(z, "z");
+    check_f32(weights, "weights");
+    check_i32(idx, "idx");
+    TORCH_CHECK(z.dim() == 2 && z.is_contiguous() && n_experts >= 1 &&
+                ff >= 1 && z.size(1) >= n_experts * ff);
+    const long T = z.size(0);
+    const int N = (int)z.size(1);
+    TORCH_CHECK(weights.dim() == 2 && weights.size(0) == T &&
+                idx.sizes() == weights.sizes());
+    Tensor out = torch::empty_like(z);
+    const bool vec = ff % 4 == 0 && N % 4 == 0 && aligned4(z) && aligned4(out);
+    launch_routed_relu2(z.data_ptr(), weights.data_ptr<float>(),
+                        idx.data_ptr<int>(), out.data_ptr(), T,
+                        (int)n_experts, (int)ff, N, (int)weights.size(1), c,
+                        vec ? 1 : 0, stream());
+    return out;
+}
+
 }  // namespace
 
 void register_moe_ops(pybind11::module_& m) {
@@ -112,4 +135,6 @@ void register_moe_ops(pybind11::module_& m) {
           "weighted sum of each token's expert outputs");
     m.def("routed_silu_glu", &routed_silu_glu,
           "silu GLU of every expert times the routing weight");
+    m.def("routed_relu2", &routed_relu2,
+          "relu(w z)^2 of every expert, relu(z)^2 of the always-on columns");
 }

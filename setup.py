@@ -35,6 +35,9 @@ ext = CUDAExtension(
         os.path.join(CSRC, "moe.hip"),
         os.path.join(CSRC, "tanh_ext.cpp"),
         os.path.join(CSRC, "tanh_stack.hip"),
+        os.path.join(CSRC, "scaled_ext.cpp"),
+        os.path.join(CSRC, "scaled.hip"),
+        os.path.join(CSRC, "ssd.hip"),
     ],
     extra_compile_args={
         "cxx": ["-O3", "-std=c++17"]
