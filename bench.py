@@ -311,6 +311,60 @@ def compare_tudatar(args) -> None:
                                     device, p_batch, p_len, d_batch, d_len)
 
 
+def compare_losivik(args) -> None:
+    """Prefill and decode throughput of a Losivik stack (windowed attention
+    with kept first tokens beside a state-space recurrence, windowed latent
+    attention, dense clamped GLU and routed relu^2 experts with a shared
+    one, a per-token side input after every layer) beside a Tudatar stack
+    (the closest family: windowed attention, latent attention, a
+    recurrence, routed experts) and the GQA-attention MoE stack, at equal
+    width, layers, heads, head and expert sizes. The recurrent state holds
+    as many numbers per head group as Tudatar's (heads x 128 x 128). The
+    window (4096) covers every context here. Random weights, synthetic
+    prompts, one GPU."""
+    from bee2bee_amd.models.hybrid import (losivik_layer_cfgs,
+                                           tudatar_layer_cfgs)
+    from bee2bee_amd.models.spec import (ModelSpec, losivik_spec,
+                                         tudatar_spec)
+
+    on_gpu = torch.cuda.is_available()
+    device = "cuda:0" if on_gpu else "cpu"
+    vocab, head_dim = 32000, 128
+    p_batch, p_len = 8, (2048 if on_gpu else 48)
+    d_batch, d_len = (64 if on_gpu else 4), (1024 if on_gpu else 32)
+    for size in args.compare_losivik.split(","):
+        z = HYBRID_SIZES[size.strip()]
+        W, H, ff, E = z["width"], z["heads"], z["ff"], z["experts"]
+        kv_rank, rot_dim, q_rank, rank = 512, 64, 768, 64
+        ssd_vdim, state, side = 64, 128, 256
+        if not on_gpu:
+            W, H, head_dim, vocab, ff, E = 64, 4, 16, 256, 32, 4
+            kv_rank, rot_dim, q_rank, rank = 24, 8, 32, 8
+            ssd_vdim, state, side = 8, 16, 8
+        common = dict(heads=H, kv_heads=max(1, H // 4), dim=head_dim,
+                      window=4096, kv_rank=kv_rank, experts=E, top_k=2,
+                      expert_ff=ff)
+        base = {"vocab": vocab, "width": W, "norm": {"eps": 1e-6},
+                "max_seq_len": 8192}
+        lo = losivik_spec(f"losivik-{size}", dict(
+            base, embedding={"scale": W ** 0.5}, token_side={"dim": side},
+            layers=losivik_layer_cfgs(
+                6, W, ssd_heads=2 * H, ssd_vdim=ssd_vdim, state=state,
+                groups=1, ff=2 * ff, keep_first=4, **common)))
+        td = tudatar_spec(f"tudatar-{size}", dict(
+            base, logit_scale=0.5, layers=tudatar_layer_cfgs(
+                6, W, rot_dim=rot_dim, q_rank=q_rank, delta_heads=H,
+                delta_kv_heads=H, delta_dim=head_dim, rank=rank, **common)))
+        dense = ModelSpec(
+            name=f"gqa-moe-{size}", vocab_size=vocab, hidden_size=W,
+            intermediate_size=ff, n_layers=6, n_heads=H,
+            n_kv_heads=max(1, H // 4), head_dim=head_dim, rope_theta=1e6,
+            max_seq_len=8192, n_experts=E, top_k_experts=2)
+        for spec in (lo, td, dense):
+            _measure_prefill_decode(spec, "losivik-vs-others", size, args,
+                                    device, p_batch, p_len, d_batch, d_len)
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -366,6 +420,16 @@ def main() -> None:
                          "stack of equal width, layers, heads and expert "
                          "sizes, at the comma-separated sizes (s, m, l); "
                          "one JSON line per size and model")
+    ap.add_argument("--compare-losivik", default=None, metavar="SIZES",
+                    help="instead of the headline run: prefill and decode "
+                         "throughput of the Losivik stack (windowed "
+                         "attention with kept first tokens beside a "
+                         "state-space recurrence, windowed latent "
+                         "attention, relu^2 experts, a token side input) "
+                         "beside a Tudatar stack and a GQA-attention MoE "
+                         "stack of equal width, layers, heads and expert "
+                         "sizes, at the comma-separated sizes (s, m, l); "
+                         "one JSON line per size and model")
     ap.add_argument("--preflight", action="store_true",
                     help="run the scale-run preflight checks (RCCL self-"
                          "test, master endpoint, env, rank wiring) and exit")
@@ -394,6 +458,9 @@ def main() -> None:
         return
     if args.compare_tudatar:
         compare_tudatar(args)
+        return
+    if args.compare_losivik:
+        compare_losivik(args)
         return
 
     from bee2bee_amd.models.spec import resolve_spec
