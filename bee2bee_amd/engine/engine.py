@@ -683,6 +683,7 @@ class InferenceEngine:
                 input_ids, positions, slots, cu_seqlens, max_len,
                 block_table=self.kv.block_table(seqs),
                 state_slots=self.kv.state_slots(seqs),
+                whole=all(start == 0 for _, _, start in chunks),
             )
         elif whole:
             hidden = self.runner.forward_prefill(

@@ -22,6 +22,13 @@ from ..models.weights import ModelWeights
 from .kv import PagedKV
 
 
+class StepMeta(tuple):
+    """What every layer of a hybrid step reads: (positions, slot_mapping,
+    cu_seqlens, seq_idx, block_table, state_slots, max_qlen). whole: every
+    chunk is known to start at position 0, so it attends to itself only."""
+    whole = False
+
+
 class Runner:
     def __init__(
         self,
@@ -397,16 +404,18 @@ class Runner:
         seq_lens: Optional[torch.Tensor] = None,
         query_lens: Optional[torch.Tensor] = None,
         state_slots: Optional[torch.Tensor] = None,
+        whole: bool = False,
     ) -> torch.Tensor:
         """Full- or chunked-prompt forward. Returns final hidden [T, H]
         (call lm_head on the rows you need). When seq_lens/query_lens are
-        given the chunk attends to the paged history (chunked prefill)."""
+        given the chunk attends to the paged history (chunked prefill).
+        whole (hybrid stacks): every chunk starts at position 0."""
         if self.spec.is_hybrid:
             # hybrid stacks always attend through the pages and carry
             # per-sequence state; returns the fp32 residual stream
             return self._forward_hybrid(
                 input_ids_or_hidden, positions, slot_mapping, cu_seqlens,
-                max_seqlen, block_table, state_slots)
+                max_seqlen, block_table, state_slots, whole)
         chunked = seq_lens is not None
 
         def attn(layer_idx, q, k, v, k_cache, v_cache):
@@ -501,6 +510,7 @@ class Runner:
         max_qlen: int,
         block_table: torch.Tensor,
         state_slots: torch.Tensor,
+        whole: bool = False,
     ) -> torch.Tensor:
         """One step of a hybrid stack over B packed chunks (prompt portions
         and single decode tokens alike). The residual stream is fp32
@@ -520,8 +530,9 @@ class Runner:
             seq_idx = torch.repeat_interleave(
                 torch.arange(B, dtype=torch.int32, device=self.device), lens,
                 output_size=T)
-        meta = (positions, slot_mapping, cu_seqlens, seq_idx, block_table,
-                state_slots, max_qlen)
+        meta = StepMeta((positions, slot_mapping, cu_seqlens, seq_idx,
+                         block_table, state_slots, max_qlen))
+        meta.whole = whole
         if s.pos_type == "sinusoid":
             x = ops.embed_sinusoid(input_ids, W.embed, s.embed_scale,
                                    positions)
@@ -882,6 +893,10 @@ class Runner:
                                              device=self.device)
         return z
 
+    # whole prompts with a chunk of at least this many tokens project keys
+    # and values instead of scoring latent rows
+    LATENT_EXPAND_MIN = 64
+
     def _latent_attn_part(self, i: int, m, ns, cols, pre, meta
                           ) -> torch.Tensor:
         """Latent attention of layer run i in absorbed form (the key
@@ -907,6 +922,16 @@ class Runner:
         ops.latent_rope_store(q[..., D:], kv, ns.kv_norm, self.spec.rms_eps,
                               C, m.rope_dims, positions, cos, sin, cache,
                               slot_mapping, m.rope_layout == "interleaved")
+        if ns.w_ukv is not None and meta.whole and \
+                max_qlen >= self.LATENT_EXPAND_MIN:
+            # keys and values of the prompt, projected from the same normed
+            # latent that was just cached
+            c = ops.slice_rmsnorm(kv, ns.kv_norm, self.spec.rms_eps)
+            kvx = F.linear(c, ns.w_ukv)
+            return ops.packed_attn(
+                q, kvx[:, : H * D].view(T, H, D),
+                kvx[:, H * D :].view(T, H, m.vdim), cu, m.scale, m.window,
+                gate, max_qlen)
         q_abs = torch.bmm(q[..., :D].transpose(0, 1), ns.w_uk)    # [H,T,C]
         lat = ops.latent_attn(q_abs, q[..., D:], gate, cache, block_table,
                               positions, seq_idx, cu, m.window, m.scale,

@@ -26,6 +26,7 @@ from typing import Dict, Iterator, Optional, Tuple
 
 import torch
 
+from ..ops import packed_attn_covers
 from .spec import ModelSpec
 
 
@@ -766,6 +767,15 @@ class ModelWeights:
             m.heads, m.vdim, m.kv_rank).transpose(1, 2))
         ns.sink = self._f32(get(q + "sink")) if m.sink else None
         ns.wo_b = None
+        # whole prompts project keys and values once instead of scoring
+        # latent rows, where that is less work and a kernel covers it
+        ns.w_ukv = None
+        if m.rot_dim == 0 and not m.sink and \
+                m.dim + m.vdim < 2 * m.kv_rank and \
+                packed_attn_covers(self.dtype, m.dim, m.vdim):
+            ns.w_ukv = torch.cat([
+                ns.w_uk.reshape(m.heads * m.dim, m.kv_rank),
+                ns.w_uv.transpose(1, 2).reshape(m.heads * m.vdim, m.kv_rank)])
 
     def _mix_ssd(self, ns, m, pre: str, q: str, get, put_in) -> None:
         rows, at = get(q + "in"), 0

@@ -667,6 +667,22 @@ def side_gate(g, table, offset: int, ids):
     return reference.side_gate(g, table, offset, ids)
 
 
+def packed_attn_covers(dtype, dim: int, vdim: int) -> bool:
+    """Shapes the packed-key prompt attention has a kernel for."""
+    return (dtype is torch.bfloat16 and dim == vdim and dim in (64, 128)
+            and hip_available())
+
+
+def packed_attn(q, k, v, cu_seqlens, scale: float, window: int, gate,
+                max_qlen: int):
+    """Whole prompts: every chunk starts at position 0 and attends to itself
+    only, so keys and values come packed instead of from pages."""
+    if _use_hip(q):
+        return require_hip().packed_attn(q, k, v, cu_seqlens, float(scale),
+                                         window, gate, max_qlen)
+    return reference.packed_attn(q, k, v, cu_seqlens, scale, window, gate)
+
+
 def ssd_scan(xbc, dt, dt_bias, rate, skip, groups: int, state, state_slots,
              cu_seqlens, positions, max_qlen: int = 0):
     """max_qlen: longest chunk of the step (host int); long chunks take the

@@ -144,7 +144,8 @@ __global__ __launch_bounds__(64) void attn_prefill_basic(
 // stride s_g): head h's output times sigmoid(head_gate[t, h]). DIST:
 // dist [2, nq] = (a, b), a_h ln(1 + b_h d) is taken off a score whose key
 // lies d positions back. KEEP: with a window, the first `keep` positions stay
-// visible to every later row (their tiles are visited first).
+// visible to every later row (their tiles are visited first). HILO on packed
+// keys applies `scale` to the fp32 scores instead of the bf16 queries.
 //
 // MODE 1 / MODE 2 split the kernel around a score buffer, for attention
 // whose scores are mixed across heads before the softmax: MODE 1 stops
@@ -173,6 +174,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
     int qt_rows = 0, long ctx = 0, float softcap = 0.f,
     const float* __restrict__ dist = nullptr, int keep = 0) {
     constexpr int KSTEPS = HD / 32;
+    constexpr bool SCALE_S = HILO && !PAGED;
     const int seq = blockIdx.z;
     const int h = blockIdx.y;
     const int kvh = h / (nq / nkv);
@@ -216,7 +218,8 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
                 short8 raw = *reinterpret_cast<const short8*>(qr + d);
 #pragma unroll
                 for (int e = 0; e < 8; ++e)
-                    a_q[ks][e] = (__bf16)(bf2f((unsigned short)raw[e]) * scale);
+                    a_q[ks][e] = (__bf16)(bf2f((unsigned short)raw[e]) *
+                                          (SCALE_S ? 1.f : scale));
             } else {
 #pragma unroll
                 for (int e = 0; e < 8; ++e) a_q[ks][e] = (__bf16)0.f;
@@ -338,6 +341,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma(
             for (int r = 0; r < 4; ++r) {
                 const int qrow = q0 + wid * PF_QROWS + lg * 4 + r;
                 const int key = kb + f * 16 + li;
+                if (SCALE_S) sfrag[f][r] *= scale;
                 if (DIST) {
                     // keys ahead of the row are masked below
                     const float d = (float)max(hist + qrow - key, 0);
@@ -561,6 +565,34 @@ extern "C" int launch_attn_prefill_paged_sink(
     else if (dist) PS_LAUNCH(64, true, false);
     else PS_LAUNCH(64, false, false);
 #undef PS_LAUNCH
+    return 0;
+}
+
+// Whole prompts on packed keys and values (each chunk starts at position 0
+// and sees only itself) with fp32-grade scores and softmax weights: the paged
+// form's options without pages. bf16, head size 64 or 128 (returns nonzero
+// otherwise); q, k, v rows of all heads side by side, row strides s_q, s_k,
+// s_v.
+extern "C" int launch_attn_prefill_packed(
+    const unsigned short* q, long s_q, const unsigned short* k, long s_k,
+    const unsigned short* v, long s_v, const int* cu, unsigned short* out,
+    long s_o, int nseq, int nq, int nkv, int hd, int max_qlen, float scale,
+    float out_scale, int window, const unsigned short* head_gate, long s_g,
+    hipStream_t stream) {
+    if (hd != 64 && hd != 128) return 1;
+    if (nseq == 0 || max_qlen == 0) return 0;
+    const dim3 grid((max_qlen + PF_TM - 1) / PF_TM, nq, nseq);
+    const int smem = prefill_mfma_smem(hd, 1);
+    const int* none = nullptr;
+#define PK_LAUNCH(HDV)                                                        \
+    hipLaunchKernelGGL((attn_prefill_mfma<HDV, false, unsigned short, true>), \
+                       grid, dim3(256), smem, stream, q, k, v, cu, none,      \
+                       none, out, nq, nkv, s_q, s_k, s_v, 0, 0, scale,        \
+                       (const float*)nullptr, out_scale, s_o, window,         \
+                       head_gate, s_g)
+    if (hd == 128) PK_LAUNCH(128);
+    else PK_LAUNCH(64);
+#undef PK_LAUNCH
     return 0;
 }
 

@@ -178,20 +178,23 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ x,
 // ------------------------------------------------------------ clamped GLU
 // [rows, 2I] -> [rows, I]: g = min(gate, L), u = clamp(up, +-L),
 // y = g * sigmoid(alpha g) * (u + 1)
-template <typename T>
+// (row, column part) grid.
+template <typename T, int VEC>
 __global__ void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ y,
-                                   long rows, long I, float limit,
-                                   float alpha) {
-    const long n = rows * I;
-    for (long idx = (long)blockIdx.x * blockDim.x + threadIdx.x; idx < n;
-         idx += (long)gridDim.x * blockDim.x) {
-        const long r = idx / I, c = idx - r * I;
-        float g = ldf(gu + r * 2 * I + c);
-        float u = ldf(gu + r * 2 * I + I + c);
-        g = fminf(g, limit);
-        u = fminf(fmaxf(u, -limit), limit);
-        stf(y + idx, g / (1.f + expf(-alpha * g)) * (u + 1.f));
+                                   long I, float limit, float alpha) {
+    const long c = ((long)blockIdx.y * blockDim.x + threadIdx.x) * VEC;
+    if (c >= I) return;             // VEC = 4 only when 4 divides I
+    const long r = blockIdx.x;
+    float gv[VEC], uv[VEC];
+    ldv<T, VEC>(gu + r * 2 * I + c, gv);
+    ldv<T, VEC>(gu + r * 2 * I + I + c, uv);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+        const float g = fminf(gv[j], limit);
+        const float u = fminf(fmaxf(uv[j], -limit), limit);
+        gv[j] = g / (1.f + expf(-alpha * g)) * (u + 1.f);
     }
+    stv<T, VEC>(y + r * I + c, gv);
 }
 
 // ------------------------------------------------------- input convolution
@@ -200,7 +203,9 @@ __global__ void clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ y,
 // sandwich layers); the short conv of a delta mixer is plain and activated.
 // h may be a column slice of a wider buffer (row stride hs); out is
 // contiguous [T, C] of type OT. Rows before the chunk come from the
-// sequence's state (its last K inputs), rows before position 0 are zero.
+// sequence's state (its last K inputs), rows before position 0 are zero. A
+// workgroup takes `per` consecutive tokens, so that the rows neighbouring
+// tokens share are fetched once.
 template <typename T, typename OT, int VEC, bool RES, bool SILU>
 __global__ void canon_conv_kernel(const T* __restrict__ h, long hs,
                                   const float* __restrict__ w,   // [K+1, C]
@@ -210,41 +215,44 @@ __global__ void canon_conv_kernel(const T* __restrict__ h, long hs,
                                   const int* __restrict__ seq_idx,
                                   const int* __restrict__ positions,
                                   OT* __restrict__ out, int C, int K,
-                                  const float* __restrict__ bias) {
-    const long t = blockIdx.x;
+                                  const float* __restrict__ bias, long Tn,
+                                  int per) {
     const int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC;
     if (c >= C) return;
-    const int b = seq_idx[t];
-    const int local = (int)t - cu[b];
-    const int pos = positions[t];
-    const long slot = state_slots[b];
-    float acc[VEC], v[VEC], wv[VEC];
-    ldv<T, VEC>(h + t * hs + c, v);
-    ldv<float, VEC>(w + (long)K * C + c, wv);
+    const long t0 = (long)blockIdx.x * per, t1 = min(t0 + per, Tn);
+    for (long t = t0; t < t1; ++t) {
+        const int b = seq_idx[t];
+        const int local = (int)t - cu[b];
+        const int pos = positions[t];
+        const long slot = state_slots[b];
+        float acc[VEC], v[VEC], wv[VEC];
+        ldv<T, VEC>(h + t * hs + c, v);
+        ldv<float, VEC>(w + (long)K * C + c, wv);
 #pragma unroll
-    for (int j = 0; j < VEC; ++j)
-        acc[j] = v[j] * (RES ? 1.f + wv[j] : wv[j]);
-    for (int d = 1; d <= K; ++d) {
-        if (pos - d < 0) break;
-        const int src = local - d;
-        if (src >= 0)
-            ldv<T, VEC>(h + (t - d) * hs + c, v);
-        else
-            ldv<T, VEC>(state + (slot * K + (K + src)) * C + c, v);
-        ldv<float, VEC>(w + (long)(K - d) * C + c, wv);
+        for (int j = 0; j < VEC; ++j)
+            acc[j] = v[j] * (RES ? 1.f + wv[j] : wv[j]);
+        for (int d = 1; d <= K; ++d) {
+            if (pos - d < 0) break;
+            const int src = local - d;
+            if (src >= 0)
+                ldv<T, VEC>(h + (t - d) * hs + c, v);
+            else
+                ldv<T, VEC>(state + (slot * K + (K + src)) * C + c, v);
+            ldv<float, VEC>(w + (long)(K - d) * C + c, wv);
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * v[j];
+            for (int j = 0; j < VEC; ++j) acc[j] += wv[j] * v[j];
+        }
+        if (bias) {
+            ldv<float, VEC>(bias + c, wv);
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) acc[j] += wv[j];
+        }
+        if (SILU) {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) acc[j] = acc[j] / (1.f + expf(-acc[j]));
+        }
+        stv<OT, VEC>(out + t * C + c, acc);
     }
-    if (bias) {
-        ldv<float, VEC>(bias + c, wv);
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) acc[j] += wv[j];
-    }
-    if (SILU) {
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) acc[j] = acc[j] / (1.f + expf(-acc[j]));
-    }
-    stv<OT, VEC>(out + t * C + c, acc);
 }
 
 // state <- the sequence's last K inputs after this chunk (thread per
@@ -529,6 +537,66 @@ qk_norm_rope_store_kernel(T* __restrict__ q, long q_tok, int H,
     }
 }
 
+// The same without a rotation, for head sizes that are multiples of 8: a
+// group of `lph` lanes (a power of two) per (token, head), eight neighbours a
+// lane. Items of a token: H query heads, G key heads, G value heads.
+template <typename T>
+__global__ void __launch_bounds__(256)
+head_norm_store_kernel(T* __restrict__ q, long q_tok, int H,
+                       const T* __restrict__ k, long k_tok, int G, int D,
+                       const float* __restrict__ wq,
+                       const float* __restrict__ wk, float eps,
+                       const float* __restrict__ q_mult,
+                       T* __restrict__ k_cache, T* __restrict__ v_cache,
+                       int bs, const int* __restrict__ slot_mapping,
+                       const T* __restrict__ v, long v_tok, int Dv, long n,
+                       int lph) {
+    const long item = (long)blockIdx.x * (256 / lph) + threadIdx.x / lph;
+    if (item >= n) return;          // whole lane groups
+    const int per = H + 2 * G;
+    const long t = item / per;
+    const int hh = (int)(item - t * per);
+    const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
+    const int g = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
+    const int size = kind == 2 ? Dv : D;
+    const int i = threadIdx.x % lph * 8;
+    const T* src = kind == 0   ? q + t * q_tok + (long)g * D
+                   : kind == 1 ? k + t * k_tok + (long)g * D
+                               : v + t * v_tok + (long)g * Dv;
+    T* dst;
+    if (kind == 0) {
+        dst = q + t * q_tok + (long)g * D;
+    } else {
+        const int slot = slot_mapping[t];
+        const long row = ((long)(slot / bs) * G + g) * bs + slot % bs;
+        dst = kind == 1 ? k_cache + row * D : v_cache + row * Dv;
+    }
+    float x[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = 0.f;
+    if (i < size) {
+        ldv<T, 4>(src + i, x);
+        ldv<T, 4>(src + i + 4, x + 4);
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += x[j] * x[j];
+    for (int off = 1; off < lph; off <<= 1) ss += __shfl_xor(ss, off);
+    if (i >= size) return;
+    if (kind != 2) {
+        const float r = (kind == 0 ? q_mult[g] : 1.f) /
+                        sqrtf(ss / (float)D + eps);
+        const float* w = (kind == 0 ? wq : wk) + i;
+        float wv[8];
+        ldv<float, 4>(w, wv);
+        ldv<float, 4>(w + 4, wv + 4);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] *= r * wv[j];
+    }
+    stv<T, 4>(dst + i, x);
+    stv<T, 4>(dst + i + 4, x + 4);
+}
+
 // ------------------------------------------------------------- launchers
 // dtype codes: 0 = bf16 (ushort bits), 1 = fp32
 
@@ -621,17 +689,21 @@ extern "C" void launch_gated_rmsnorm(const float* x, const float* w,
 extern "C" void launch_clamped_glu(const void* gu, void* y, long rows, long I,
                                    float limit, float alpha, int f32,
                                    hipStream_t s) {
-    const long n = rows * I;
-    if (n == 0) return;
+    if (rows * I == 0) return;
     const int th = 256;
-    long blocks = (n + th - 1) / th;
-    if (blocks > 65536) blocks = 65536;
-    if (f32)
-        clamped_glu_kernel<float><<<(int)blocks, th, 0, s>>>(
-            (const float*)gu, (float*)y, rows, I, limit, alpha);
-    else
-        clamped_glu_kernel<unsigned short><<<(int)blocks, th, 0, s>>>(
-            (const unsigned short*)gu, (unsigned short*)y, rows, I, limit, alpha);
+    // contiguous torch buffers: a multiple of 4 keeps every row aligned
+    const bool vec = I % 4 == 0 && (uintptr_t)gu % 16 == 0 &&
+                     (uintptr_t)y % 16 == 0;
+    const long per = th * (vec ? 4 : 1);
+    const dim3 grid((unsigned)rows, (unsigned)((I + per - 1) / per));
+#define CG_LAUNCH(TT, V)                                                      \
+    hipLaunchKernelGGL((clamped_glu_kernel<TT, V>), grid, dim3(th), 0, s,     \
+                       (const TT*)gu, (TT*)y, I, limit, alpha)
+    if (f32 && vec) CG_LAUNCH(float, 4);
+    else if (f32) CG_LAUNCH(float, 1);
+    else if (vec) CG_LAUNCH(unsigned short, 4);
+    else CG_LAUNCH(unsigned short, 1);
+#undef CG_LAUNCH
 }
 
 template <typename T, typename OT, bool RES, bool SILU>
@@ -643,15 +715,17 @@ static void conv_dispatch(const void* h, long hs, const float* w, void* state,
     const int th = C >= 256 ? 256 : 64;
     const int vec = vec4 ? 4 : 1;
     const int lanes = (C + vec - 1) / vec;
-    const dim3 g1((unsigned)T_, (lanes + th - 1) / th), g2(B, (C + th - 1) / th);
+    const int per = T_ >= 4096 ? 8 : 1;
+    const dim3 g1((unsigned)((T_ + per - 1) / per), (lanes + th - 1) / th),
+        g2(B, (C + th - 1) / th);
     if (vec4)
         canon_conv_kernel<T, OT, 4, RES, SILU><<<g1, th, 0, s>>>(
             (const T*)h, hs, w, (const T*)state, state_slots, cu, seq_idx,
-            positions, (OT*)out, C, K, bias);
+            positions, (OT*)out, C, K, bias, T_, per);
     else
         canon_conv_kernel<T, OT, 1, RES, SILU><<<g1, th, 0, s>>>(
             (const T*)h, hs, w, (const T*)state, state_slots, cu, seq_idx,
-            positions, (OT*)out, C, K, bias);
+            positions, (OT*)out, C, K, bias, T_, per);
     if (K > 0)
         canon_state_kernel<T><<<g2, th, 0, s>>>(
             (const T*)h, hs, (T*)state, state_slots, cu, C, K);
@@ -783,6 +857,27 @@ extern "C" int launch_qk_norm_rope_store(
     int f32, hipStream_t s) {
     if (D > QKN_MAXD) return 1;
     if (T == 0) return 0;
+    const long unit = f32 ? 16 : 8;         // bytes of four elements
+    const auto ok = [&](const void* p, long stride) {
+        return (uintptr_t)p % unit == 0 && stride % 4 == 0;
+    };
+    if (dims == 0 && v && D % 8 == 0 && Dv % 8 == 0 && Dv <= QKN_MAXD &&
+        ok(q, q_tok) && ok(k, k_tok) && ok(v, v_tok) && ok(k_cache, 0) &&
+        ok(v_cache, 0) && (uintptr_t)wq % 16 == 0 && (uintptr_t)wk % 16 == 0) {
+        const long n = T * (H + 2 * G);
+        int lph = 1;
+        while (lph * 8 < D || lph * 8 < Dv) lph <<= 1;
+        const unsigned blocks = (unsigned)((n + 256 / lph - 1) / (256 / lph));
+#define HN_LAUNCH(TT)                                                         \
+    hipLaunchKernelGGL((head_norm_store_kernel<TT>), dim3(blocks), dim3(256), \
+                       0, s, (TT*)q, q_tok, H, (const TT*)k, k_tok, G, D, wq, \
+                       wk, eps, q_mult, (TT*)k_cache, (TT*)v_cache, bs,       \
+                       slot_mapping, (const TT*)v, v_tok, Dv, n, lph)
+        if (f32) HN_LAUNCH(float);
+        else HN_LAUNCH(unsigned short);
+#undef HN_LAUNCH
+        return 0;
+    }
     if (f32)
         qk_norm_rope_store_kernel<float><<<T, 256, 0, s>>>(
             (float*)q, q_tok, H, (const float*)k, k_tok, G, D, wq, wk, eps,

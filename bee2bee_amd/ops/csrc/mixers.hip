@@ -1291,6 +1291,7 @@ extern "C" int launch_latent_attn_mfma(
         if (ksteps <= 4) LM_CASE(4, true, 256);
         else if (ksteps <= 8) LM_CASE(8, true, 256);
         else if (ksteps <= 12) LM_CASE(12, true, 256);
+        else if (ksteps <= 16) LM_CASE(16, true, 256);
         else LM_CASE(18, true, 256);
         if (splits > 1) {
             const dim3 g2(Tn, H);
@@ -1305,6 +1306,7 @@ extern "C" int launch_latent_attn_mfma(
     if (ksteps <= 4) LM_CASE(4, false, 256);
     else if (ksteps <= 8) LM_CASE(8, false, 256);
     else if (ksteps <= 12) LM_CASE(12, false, 256);
+    else if (ksteps <= 16) LM_CASE(16, false, 256);
     else LM_CASE(18, false, 256);
     return 0;
 }

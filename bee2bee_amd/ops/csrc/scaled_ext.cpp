@@ -27,11 +27,18 @@ void launch_side_gate(const void*, const void*, long, long, const long*,
 void launch_gated_group_norm(const float*, long, const void*, long,
                              const float*, void*, long, long, int, int, float,
                              float, int, int, hipStream_t);
+int launch_attn_prefill_packed(const unsigned short*, long,
+                               const unsigned short*, long,
+                               const unsigned short*, long, const int*,
+                               unsigned short*, long, int, int, int, int, int,
+                               float, float, int, const unsigned short*, long,
+                               hipStream_t);
 int ssd_piece_tokens();
 int launch_ssd_scan(const void*, long, const void*, long, const float*,
                     const float*, const float*, float*, const int*,
-                    const int*, const int*, float*, float*, float*, int, int,
-                    int, int, int, int, int, int, hipStream_t);
+                    const int*, const int*, float*, float*, double*, float*,
+                    float*, float*, int*, int, int, int, int, int, int, int,
+                    int, hipStream_t);
 }
 
 namespace {
@@ -256,26 +263,74 @@ Tensor ssd_scan(const Tensor& xbc, const Tensor& dt, const Tensor& dt_bias,
     // portions past this length: 64-token pieces in parallel. `pieces`
     // bounds the batch's piece count without reading the lengths.
     long pieces = 0;
-    Tensor ws, fade;
-    float *wp = nullptr, *fp = nullptr;
+    Tensor ws, logs, per_tok, fade, table;
+    float *wp = nullptr, *steps = nullptr, *tails = nullptr, *fp = nullptr;
+    double* lp = nullptr;
+    int* tp = nullptr;
     if (max_qlen > 16) {
-        pieces = T / ssd_piece_tokens() + B;
+        const long L = ssd_piece_tokens();
+        pieces = T / L + B;
         ws = torch::empty({pieces, (long)H, (long)N, (long)V}, f32opt);
+        logs = torch::empty({pieces, (long)H, L},
+                            f32opt.dtype(torch::kFloat64));
+        per_tok = torch::empty({2, pieces, (long)H, L}, f32opt);
         fade = torch::empty({pieces, (long)H}, f32opt);
+        table = torch::empty({pieces, 2}, f32opt.dtype(torch::kInt32));
         wp = ws.data_ptr<float>();
+        lp = logs.data_ptr<double>();
+        steps = per_tok.data_ptr<float>();
+        tails = steps + pieces * H * L;
         fp = fade.data_ptr<float>();
+        tp = table.data_ptr<int>();
     }
-    const bool vec = N % 4 == 0 && V % 4 == 0 && aligned4(xbc) &&
-                     aligned4(state.view({-1}));
+    const bool vec = N % 4 == 0 && V % 4 == 0 && xbc.stride(0) % 4 == 0 &&
+                     reinterpret_cast<uintptr_t>(xbc.data_ptr()) % 16 == 0 &&
+                     reinterpret_cast<uintptr_t>(state.data_ptr()) % 16 == 0;
     const int rc = launch_ssd_scan(
         xbc.data_ptr(), xbc.stride(0), dt.data_ptr(), dt.stride(0),
         dt_bias.data_ptr<float>(), rate.data_ptr<float>(),
         skip.data_ptr<float>(), state.data_ptr<float>(),
         state_slots.data_ptr<int>(), cu.data_ptr<int>(),
-        positions.data_ptr<int>(), y.data_ptr<float>(), wp, fp, (int)pieces,
-        B, H, G, N, V, c, vec ? 1 : 0, stream());
+        positions.data_ptr<int>(), y.data_ptr<float>(), wp, lp, steps, tails,
+        fp, tp, (int)pieces, B, H, G, N, V, c, vec ? 1 : 0, stream());
     TORCH_CHECK(rc == 0, "ssd_scan: state size must be <= 512");
     return y;
+}
+
+// q [T, H, D], k, v [T, G, D]: rows whose heads lie side by side (bf16, D 64
+// or 128); gate [T, H] raw or none -> [T, H * D]
+Tensor packed_attn(const Tensor& q, const Tensor& k, const Tensor& v,
+                   const Tensor& cu, double scale, int64_t window,
+                   const std::optional<Tensor>& gate, int64_t max_qlen) {
+    check_i32(cu, "cu_seqlens");
+    TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && v.sizes() == k.sizes() &&
+                window >= 0 && max_qlen >= 1);
+    const long T = q.size(0);
+    const int H = (int)q.size(1), D = (int)q.size(2), G = (int)k.size(1);
+    TORCH_CHECK(k.size(0) == T && k.size(2) == D && G >= 1 && H % G == 0);
+    for (const Tensor* t : {&q, &k, &v})
+        TORCH_CHECK(t->is_cuda() && t->scalar_type() == torch::kBFloat16 &&
+                        t->stride(2) == 1 && t->stride(1) == D &&
+                        t->stride(0) % 8 == 0 &&
+                        reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0,
+                    "packed_attn: bf16 rows on 16-byte boundaries");
+    const unsigned short* gp = nullptr;
+    long gs = 0;
+    if (gate.has_value()) {
+        check_slice(*gate, T, H, torch::kBFloat16, "gate");
+        gp = (const unsigned short*)gate->data_ptr();
+        gs = gate->stride(0);
+    }
+    Tensor out = torch::empty({T, (long)H * D}, q.options());
+    const int rc = launch_attn_prefill_packed(
+        (const unsigned short*)q.data_ptr(), q.stride(0),
+        (const unsigned short*)k.data_ptr(), k.stride(0),
+        (const unsigned short*)v.data_ptr(), v.stride(0), cu.data_ptr<int>(),
+        (unsigned short*)out.data_ptr(), out.stride(0), (int)cu.numel() - 1,
+        H, G, D, (int)max_qlen, (float)scale, 1.f, (int)window, gp, gs,
+        stream());
+    TORCH_CHECK(rc == 0, "packed_attn: head size must be 64 or 128");
+    return out;
 }
 
 }  // namespace
@@ -290,6 +345,8 @@ void register_scaled_ops(pybind11::module_& m) {
     m.def("side_gate", &side_gate, "gelu_tanh(g) * token side row");
     m.def("gated_group_norm", &gated_group_norm,
           "group_norm(y * silu(z)) * w into a column slice");
+    m.def("packed_attn", &packed_attn,
+          "windowed causal attention of whole prompts on packed keys");
     m.def("ssd_scan", &ssd_scan,
           "state-space recurrence with carried fp32 state");
 }

@@ -10,19 +10,23 @@
 //  * ssd_serial: decode rows and short portions. A workgroup keeps a 64-column
 //    slice of one (sequence, head) state in registers and walks the tokens.
 //  * chunk-parallel, for long portions, in pieces of 64 tokens:
+//    ssd_prep     piece table, step sizes d and running log decays A;
 //    ssd_states   what a piece adds to the state, sum_t exp(A_L - A_t) d_t
-//                 B_t x_t^T, A the running log decay inside the piece;
+//                 B_t x_t^T;
 //    ssd_carry    walks the pieces of each (sequence, head) in order, turning
 //                 those into the state at every piece's start;
 //    ssd_outputs  y = (C B^T . exp(A_t - A_s) d_s, s <= t) X + exp(A_t) C S.
-//    All products run on v_mfma_f32_16x16x4_f32: fp32 operands and sums, for
-//    bf16 and fp32 activations alike. Running log decays are kept in fp64, so
-//    that their differences hold fp32 precision however far they run.
+//    Products with an fp32 operand run on v_mfma_f32_16x16x4_f32, fp32 sums,
+//    for bf16 and fp32 activations alike; C B^T of bf16 activations runs on
+//    v_mfma_f32_16x16x32_bf16 (its products are exact). Running log decays
+//    are kept in fp64, so that their differences hold fp32 precision however
+//    far they run.
 //
 // Fragment maps of v_mfma_f32_16x16x4_f32: A: lane -> row l & 15, k = l >> 4;
 // B: lane -> column l & 15, k = l >> 4; C: column l & 15, rows (l >> 4) * 4 +
 // r. Which four k values a step takes is free as long as A and B agree: where
-// a lane reads four neighbours at once, step e of four takes k = 4 (l >> 4) + e.
+// a lane reads E neighbours at once, step e of E takes k = E (l >> 4) + e. With
+// E = 8 the same registers are an A or B fragment of the bf16 instruction.
 #include "common.h"
 
 namespace {
@@ -45,19 +49,56 @@ template <> DEV_INLINE void ld4<unsigned short>(const unsigned short* p,
     o[2] = bf2f((unsigned short)(w.y & 0xffffu));
     o[3] = bf2f((unsigned short)(w.y >> 16));
 }
-// four neighbours at column c of a row of n; zeros past its end
-template <typename T, bool VEC>
-DEV_INLINE void ld4_row(const T* row, int c, int n, float* o) {
-    if (VEC) {                      // n is a multiple of 4: all or none
-        if (c < n) {
-            ld4<T>(row + c, o);
+// eight neighbours at column c of a row of n; zeros past its end. VEC: n is a
+// multiple of 8 and the addresses are aligned.
+template <typename T> struct Row8;
+template <> struct Row8<unsigned short> {
+    short8 v;
+    template <bool VEC>
+    DEV_INLINE void load(const unsigned short* row, int c, int n) {
+        v = short8{0, 0, 0, 0, 0, 0, 0, 0};
+        if (VEC) {
+            if (c < n) v = *reinterpret_cast<const short8*>(row + c);
         } else {
-            o[0] = o[1] = o[2] = o[3] = 0.f;
-        }
-    } else {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o[e] = c + e < n ? ldf(row + c + e) : 0.f;
+            for (int e = 0; e < 8; ++e)
+                if (c + e < n) v[e] = (short)row[c + e];
+        }
     }
+    DEV_INLINE float get(int e) const { return bf2f((unsigned short)v[e]); }
+};
+template <> struct Row8<float> {
+    float v[8];
+    template <bool VEC>
+    DEV_INLINE void load(const float* row, int c, int n) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = 0.f;
+        if (VEC) {
+            if (c < n) {
+                ld4<float>(row + c, v);
+                ld4<float>(row + c + 4, v + 4);
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e)
+                if (c + e < n) v[e] = row[c + e];
+        }
+    }
+    DEV_INLINE float get(int e) const { return v[e]; }
+};
+// acc += A B^T over the 32 columns that the lanes' pieces of both cover
+DEV_INLINE f32x4 mma32(const Row8<unsigned short>& a,
+                       const Row8<unsigned short>& b, f32x4 acc) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+        __builtin_bit_cast(bf16x8, a.v), __builtin_bit_cast(bf16x8, b.v), acc,
+        0, 0, 0);
+}
+DEV_INLINE f32x4 mma32(const Row8<float>& a, const Row8<float>& b, f32x4 acc) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.v[e], b.v[e], acc, 0, 0,
+                                                   0);
+    return acc;
 }
 
 DEV_INLINE float softplus_f(float z) {
@@ -77,8 +118,13 @@ struct SsdArgs {
     const int* cu;
     const int* positions;
     float* y;               // [Tn, H * V]
-    float* ws;              // chunk form: [pieces, H, N, V]
-    float* fade;            // chunk form: [pieces, H]
+    // chunk form
+    float* ws;              // [pieces, H, N, V]
+    double* logs;           // [pieces, H, 64] running log decay A
+    float* steps;           // [pieces, H, 64] d
+    float* tails;           // [pieces, H, 64] d exp(A_L - A), 0 past the end
+    float* fade;            // [pieces, H] exp(A_L)
+    int* table;             // [pieces, 2] first row, rows (0: no such piece)
     int B, H, G, N, V;
 };
 
@@ -228,96 +274,98 @@ DEV_INLINE void sd_decay(const SsdArgs& a, int h, int lo, int n, int lane,
     *A = s;
 }
 
-constexpr int SD_NS = 128;       // state rows per workgroup of ssd_states
-constexpr int SD_BS = SD_NS + 16;    // LDS row strides: the four k rows a
-constexpr int SD_XS = SD_L + 16;     // fragment read touches sit 16 banks apart
+// wave per (piece, head)
+template <typename T>
+__global__ void __launch_bounds__(SD_THREADS) ssd_prep_kernel(SsdArgs a) {
+    int lo = 0, n = 0;
+    const bool ok = sd_piece(a.cu, a.B, blockIdx.x, &lo, &n);
+    if (threadIdx.x == 0 && blockIdx.y == 0) {
+        a.table[2 * blockIdx.x] = lo;
+        a.table[2 * blockIdx.x + 1] = ok ? n : 0;
+    }
+    const int h = blockIdx.y * (SD_THREADS / WAVE) + threadIdx.x / WAVE;
+    if (!ok || h >= a.H) return;
+    const int lane = threadIdx.x % WAVE;
+    float d;
+    double A;
+    sd_decay<T>(a, h, lo, n, lane, &d, &A);
+    const double last = __shfl(A, WAVE - 1);
+    const long row = (long)blockIdx.x * a.H + h, at = row * SD_L + lane;
+    a.logs[at] = A;
+    a.steps[at] = d;
+    a.tails[at] = d * expf((float)(last - A));
+    if (lane == 0) a.fade[row] = expf((float)last);
+}
 
-// (piece, head, 128-row x 64-column block of the state); a wave owns every
-// fourth 16-row tile against all the block's columns.
-template <typename T, int VT, bool VEC>
+// (piece, head, 128-row x 64-column block of the state); a wave owns two
+// 16-row tiles against all the block's columns.
+constexpr int SD_NT = 2;
+constexpr int SD_NS = SD_NT * 16 * (SD_THREADS / WAVE);
+
+template <typename T, int VT>
 __global__ void __launch_bounds__(SD_THREADS)
 ssd_states_kernel(SsdArgs a) {
-    __shared__ float bs[SD_L * SD_BS];
-    __shared__ float xs[SD_L * SD_XS];
-    __shared__ float wt[SD_L];
-    int lo, n;
-    if (!sd_piece(a.cu, a.B, blockIdx.x, &lo, &n)) return;
+    const int lo = a.table[2 * blockIdx.x], n = a.table[2 * blockIdx.x + 1];
+    if (n == 0) return;
     const int h = blockIdx.y, g = h / (a.H / a.G);
     const int vblk = (a.V + SD_L - 1) / SD_L;
-    const int n0 = blockIdx.z / vblk * SD_NS, v0 = blockIdx.z % vblk * SD_L;
-    const int tid = threadIdx.x, lane = tid % WAVE;
-    const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
+    const int lane = threadIdx.x % WAVE;
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+    const int lg = lane >> 4, li = lane & 15;
     const int N = a.N, V = a.V;
-    if (wid == 0) {
-        float d;
-        double A;
-        sd_decay<T>(a, h, lo, n, lane, &d, &A);
-        const double last = __shfl(A, WAVE - 1);
-        wt[lane] = d * expf((float)(last - A));
-        if (lane == 0 && blockIdx.z == 0)
-            a.fade[(long)blockIdx.x * a.H + h] = expf((float)last);
-    }
-    __syncthreads();
+    const int n0 = blockIdx.z / vblk * SD_NS + wid * SD_NT * 16;
+    const int v0 = blockIdx.z % vblk * SD_L;
+    if (n0 >= N) return;                // no workgroup barrier below
+    // columns past the end repeat the last one and are not stored
     const T* X = (const T*)a.xbc + (long)h * V;
     const T* Bp = (const T*)a.xbc + (long)a.H * V + (long)g * N;
-    // rows past the end repeat the last one; their weight is zero
-    constexpr int BU = SD_NS / 4, XU = SD_L / 4;
-    const int nlive = min(SD_NS, (N - n0 + 15) / 16 * 16);
-    for (int i = tid; i < SD_L * BU; i += SD_THREADS) {
-        const int t = i / BU, c = (i - t * BU) * 4;
-        if (c >= nlive) continue;
-        float v[4];
-        ld4_row<T, VEC>(Bp + (long)(lo + min(t, n - 1)) * a.xs, n0 + c, N, v);
-        const float w = wt[t];
+    int xc[VT], bc[SD_NT];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) bs[t * SD_BS + c + e] = w * v[e];
-    }
-    for (int i = tid; i < SD_L * XU; i += SD_THREADS) {
-        const int t = i / XU, c = (i - t * XU) * 4;
-        if (c >= VT * 16) continue;
-        float v[4];
-        ld4_row<T, VEC>(X + (long)(lo + min(t, n - 1)) * a.xs, v0 + c, V, v);
+    for (int v = 0; v < VT; ++v) xc[v] = min(v0 + v * 16 + li, V - 1);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) xs[t * SD_XS + c + e] = v[e];
-    }
-    __syncthreads();
-    const int lg = lane >> 4, li = lane & 15;
-    constexpr int NT = SD_NS / 16 / (SD_THREADS / WAVE);    // row tiles a wave
-    f32x4 acc[NT][VT];
+    for (int i = 0; i < SD_NT; ++i) bc[i] = min(n0 + i * 16 + li, N - 1);
+    const float* tail = a.tails + ((long)blockIdx.x * a.H + h) * SD_L;
+    f32x4 acc[SD_NT][VT];
 #pragma unroll
-    for (int i = 0; i < NT; ++i)
+    for (int i = 0; i < SD_NT; ++i)
 #pragma unroll
         for (int v = 0; v < VT; ++v) acc[i][v] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < SD_L; k += 4) {
-        float xb[VT];
+    // rows past the end repeat the last one; their weight is zero
+    const int kend = (n + 15) / 16 * 16;
+    for (int k0 = 0; k0 < kend; k0 += 16) {
+        float xv[4][VT], bv[4][SD_NT];
 #pragma unroll
-        for (int v = 0; v < VT; ++v)
-            xb[v] = xs[(k + lg) * SD_XS + v * 16 + li];
+        for (int u = 0; u < 4; ++u) {
+            const int t = k0 + u * 4 + lg;
+            const long row = (long)(lo + min(t, n - 1)) * a.xs;
+            const float w = tail[t];
 #pragma unroll
-        for (int i = 0; i < NT; ++i) {
-            const int nt = i * (SD_THREADS / WAVE) + wid;
-            if (nt * 16 >= nlive) continue;
-            const float ba = bs[(k + lg) * SD_BS + nt * 16 + li];
+            for (int v = 0; v < VT; ++v) xv[u][v] = ldf(X + row + xc[v]);
 #pragma unroll
-            for (int v = 0; v < VT; ++v)
-                acc[i][v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    ba, xb[v], acc[i][v], 0, 0, 0);
+            for (int i = 0; i < SD_NT; ++i)
+                bv[u][i] = ldf(Bp + row + bc[i]) * w;
         }
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int i = 0; i < SD_NT; ++i)
+#pragma unroll
+                for (int v = 0; v < VT; ++v)
+                    acc[i][v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                        bv[u][i], xv[u][v], acc[i][v], 0, 0, 0);
     }
     float* out = a.ws + ((long)blockIdx.x * a.H + h) * N * V;
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-        const int nt = i * (SD_THREADS / WAVE) + wid;
+    for (int i = 0; i < SD_NT; ++i)
 #pragma unroll
-        for (int v = 0; v < VT; ++v) {
-            const int c = v0 + v * 16 + li;
+        for (int r = 0; r < 4; ++r) {
+            const int row = n0 + i * 16 + lg * 4 + r;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                const int row = n0 + nt * 16 + lg * 4 + r;
+            for (int v = 0; v < VT; ++v) {
+                const int c = v0 + v * 16 + li;
                 if (row < N && c < V) out[(long)row * V + c] = acc[i][v][r];
             }
         }
-    }
 }
 
 // per (sequence, head), VW state elements a thread: replace each piece's own
@@ -374,77 +422,82 @@ ssd_carry_kernel(SsdArgs a) {
 }
 
 // (piece, head, 64-column block); wave w owns token rows 16w .. 16w+15 of the
-// piece and needs no other wave's results. MS: LDS row stride of its masked
-// C B^T tile, in the C layout's rows and read back as the A operand.
+// piece and needs no other wave's results. SD_MS: LDS row stride of its masked
+// C B^T tile, written in the C layout and read back as the A operand.
 constexpr int SD_MS = SD_L + 4;
+
+// what one step of 32 state rows reads: C of the wave's tokens, B of the
+// tokens up to them, the state
+template <typename T, int VT> struct SdStep {
+    Row8<T> c, b[4];
+    float s[VT][8];
+};
 
 template <typename T, int VT, bool VEC>
 __global__ void __launch_bounds__(SD_THREADS)
 ssd_outputs_kernel(SsdArgs a) {
     __shared__ __attribute__((aligned(16))) float ms[SD_THREADS / WAVE]
                                                     [16 * SD_MS];
-    __shared__ double As[SD_L];
-    __shared__ float ds[SD_L];
-    int lo, n;
-    if (!sd_piece(a.cu, a.B, blockIdx.x, &lo, &n)) return;
-    const int h = blockIdx.y, g = h / (a.H / a.G);
-    const int v0 = blockIdx.z * SD_L;
-    const int tid = threadIdx.x, lane = tid % WAVE;
-    const int wid = __builtin_amdgcn_readfirstlane(tid / WAVE);
-    const int lg = lane >> 4, li = lane & 15;
-    const int N = a.N, V = a.V;
-    if (wid == 0) {
-        float d;
-        double A;
-        sd_decay<T>(a, h, lo, n, lane, &d, &A);
-        As[lane] = A;
-        ds[lane] = d;
-    }
-    __syncthreads();
+    const int lo = a.table[2 * blockIdx.x], n = a.table[2 * blockIdx.x + 1];
+    const int lane = threadIdx.x % WAVE;
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
     const int t0 = wid * 16;
     if (t0 >= n) return;                // no workgroup barrier below
+    const int h = blockIdx.y, g = h / (a.H / a.G);
+    const int v0 = blockIdx.z * SD_L;
+    const int lg = lane >> 4, li = lane & 15;
+    const int N = a.N, V = a.V;
+    const long hp = (long)blockIdx.x * a.H + h;
     const T* X = (const T*)a.xbc + (long)h * V;
     const T* Bp = (const T*)a.xbc + (long)a.H * V + (long)g * N;
-    const T* Cp = Bp + (long)a.G * N;
-    const T* crow = Cp + (long)(lo + min(t0 + li, n - 1)) * a.xs;
-    const float* S = a.ws + ((long)blockIdx.x * a.H + h) * N * V;
+    const T* crow = Bp + (long)a.G * N + (long)(lo + min(t0 + li, n - 1)) * a.xs;
+    const T* brow[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+        brow[j] = Bp + (long)(lo + min(j * 16 + li, n - 1)) * a.xs;
+    const float* S = a.ws + hp * N * V;
+    // columns past the end repeat the last one and are not stored
+    int col[VT];
+#pragma unroll
+    for (int v = 0; v < VT; ++v) col[v] = min(v0 + v * 16 + li, V - 1);
 
+    auto load = [&](SdStep<T, VT>& st, int k) {
+        const int kc = k + lg * 8;
+        st.c.template load<VEC>(crow, kc, N);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)     // later keys than any row: unused
+            if (j <= wid) st.b[j].template load<VEC>(brow[j], kc, N);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            // rows past the end repeat the last one; C is zero there
+            const float* srow = S + (long)min(kc + e, N - 1) * V;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) st.s[v][e] = srow[col[v]];
+        }
+    };
     f32x4 acc[VT], cb[4];
 #pragma unroll
     for (int v = 0; v < VT; ++v) acc[v] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int j = 0; j < 4; ++j) cb[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    // C S and C B^T share the C fragments
-    for (int k = 0; k < N; k += 16) {
-        const int kc = k + lg * 4;
-        float c[4];
-        ld4_row<T, VEC>(crow, kc, N, c);
+    SdStep<T, VT> cur, nxt;
+    load(cur, 0);
+    for (int k = 0; k < N; k += 32) {
+        if (k + 32 < N) load(nxt, k + 32);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            if (j > wid) continue;      // keys after every row of the wave
-            float bb[4];
-            ld4_row<T, VEC>(Bp + (long)(lo + min(j * 16 + li, n - 1)) * a.xs,
-                            kc, N, bb);
+        for (int j = 0; j < 4; ++j)
+            if (j <= wid) cb[j] = mma32(cur.c, cur.b[j], cb[j]);
 #pragma unroll
-            for (int e = 0; e < 4; ++e)
-                cb[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(c[e], bb[e],
-                                                             cb[j], 0, 0, 0);
-        }
+        for (int e = 0; e < 8; ++e)
 #pragma unroll
-        for (int v = 0; v < VT; ++v) {
-            const int col = v0 + v * 16 + li;
-            float s[4];
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
-                s[e] = kc + e < N && col < V ? S[(long)(kc + e) * V + col]
-                                             : 0.f;
-#pragma unroll
-            for (int e = 0; e < 4; ++e)
+            for (int v = 0; v < VT; ++v)
                 acc[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    c[e], s[e], acc[v], 0, 0, 0);
-        }
+                    cur.c.get(e), cur.s[v][e], acc[v], 0, 0, 0);
+        cur = nxt;
     }
     float* m = ms[wid];
+    const double* As = a.logs + hp * SD_L;
+    const float* ds = a.steps + hp * SD_L;
     double At[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -472,31 +525,32 @@ ssd_outputs_kernel(SsdArgs a) {
         if (j > wid) continue;
         const f32x4 mv = *reinterpret_cast<const f32x4*>(
             m + li * SD_MS + j * 16 + lg * 4);
+        float x[4][VT];
 #pragma unroll
-        for (int v = 0; v < VT; ++v) {
-            const int col = v0 + v * 16 + li;
+        for (int e = 0; e < 4; ++e) {
+            const long row =
+                (long)(lo + min(j * 16 + lg * 4 + e, n - 1)) * a.xs;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int s = min(j * 16 + lg * 4 + e, n - 1);
-                const float x =
-                    col < V ? ldf(X + (long)(lo + s) * a.xs + col) : 0.f;
-                acc[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    mv[e], x, acc[v], 0, 0, 0);
-            }
+            for (int v = 0; v < VT; ++v) x[e][v] = ldf(X + row + col[v]);
         }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int v = 0; v < VT; ++v)
+                acc[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    mv[e], x[e][v], acc[v], 0, 0, 0);
     }
     const float skip = a.skip[h];
 #pragma unroll
-    for (int v = 0; v < VT; ++v) {
-        const int col = v0 + v * 16 + li;
-        if (col >= V) continue;
+    for (int r = 0; r < 4; ++r) {
+        const int t = t0 + lg * 4 + r;
+        if (t >= n) continue;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int t = t0 + lg * 4 + r;
-            if (t >= n) continue;
-            const float x = ldf(X + (long)(lo + t) * a.xs + col);
-            a.y[(long)(lo + t) * a.H * V + (long)h * V + col] =
-                acc[v][r] + skip * x;
+        for (int v = 0; v < VT; ++v) {
+            const float x = ldf(X + (long)(lo + t) * a.xs + col[v]);
+            if (v0 + v * 16 + li < V)
+                a.y[(long)(lo + t) * a.H * V + (long)h * V + col[v]] =
+                    acc[v][r] + skip * x;
         }
     }
 }
@@ -534,31 +588,32 @@ int ssd_dispatch(const SsdArgs& a, int pieces, bool vec, hipStream_t s) {
     const long per = SD_THREADS * (cv ? 4 : 1);
     const dim3 gc(a.B, a.H, (unsigned)((NV + per - 1) / per));
     const int vt = a.V <= 16 ? 1 : a.V <= 32 ? 2 : 4;
-#define SD_RUN(K, VT, GRID)                                                   \
-    do {                                                                      \
-        if (vec)                                                              \
-            hipLaunchKernelGGL((K<T, VT, true>), GRID, dim3(SD_THREADS), 0,   \
-                               s, a);                                         \
-        else                                                                  \
-            hipLaunchKernelGGL((K<T, VT, false>), GRID, dim3(SD_THREADS), 0,  \
-                               s, a);                                         \
-    } while (0)
-#define SD_VT(K, GRID)                                                        \
-    do {                                                                      \
-        if (vt == 1) SD_RUN(K, 1, GRID);                                      \
-        else if (vt == 2) SD_RUN(K, 2, GRID);                                 \
-        else SD_RUN(K, 4, GRID);                                              \
-    } while (0)
-    SD_VT(ssd_states_kernel, gs);
+    const dim3 gp(pieces, (a.H + SD_THREADS / WAVE - 1) / (SD_THREADS / WAVE));
+    hipLaunchKernelGGL((ssd_prep_kernel<T>), gp, dim3(SD_THREADS), 0, s, a);
+#define SD_STATES(VT)                                                         \
+    hipLaunchKernelGGL((ssd_states_kernel<T, VT>), gs, dim3(SD_THREADS), 0, s, \
+                       a)
+    if (vt == 1) SD_STATES(1);
+    else if (vt == 2) SD_STATES(2);
+    else SD_STATES(4);
+#undef SD_STATES
     if (cv)
         hipLaunchKernelGGL((ssd_carry_kernel<4>), gc, dim3(SD_THREADS), 0, s,
                            a);
     else
         hipLaunchKernelGGL((ssd_carry_kernel<1>), gc, dim3(SD_THREADS), 0, s,
                            a);
-    SD_VT(ssd_outputs_kernel, go);
-#undef SD_VT
-#undef SD_RUN
+#define SD_OUTPUTS(VT, VC)                                                    \
+    hipLaunchKernelGGL((ssd_outputs_kernel<T, VT, VC>), go, dim3(SD_THREADS), \
+                       0, s, a)
+    const bool v8 = vec && a.N % 8 == 0 && a.V % 8 == 0 && a.xs % 8 == 0;
+    if (vt == 1 && v8) SD_OUTPUTS(1, true);
+    else if (vt == 1) SD_OUTPUTS(1, false);
+    else if (vt == 2 && v8) SD_OUTPUTS(2, true);
+    else if (vt == 2) SD_OUTPUTS(2, false);
+    else if (v8) SD_OUTPUTS(4, true);
+    else SD_OUTPUTS(4, false);
+#undef SD_OUTPUTS
     return 0;
 }
 
@@ -567,20 +622,23 @@ int ssd_dispatch(const SsdArgs& a, int pieces, bool vec, hipStream_t s) {
 extern "C" int ssd_piece_tokens() { return SD_L; }
 
 // pieces 0: token-serial form; else an upper bound of the number of 64-token
-// pieces in the batch, ws [pieces, H, N, V] and fade [pieces, H] sized for
-// it. c: 0 = bf16, 1 = fp32 activations. vec: N, V, xs and the addresses
-// allow 4-element accesses. Returns nonzero when the state size is above 512.
+// pieces in the batch, ws, logs, steps, tails, fade and table (see SsdArgs)
+// sized for it. c: 0 = bf16, 1 = fp32 activations. vec: N, V and xs allow
+// 4-element accesses, xbc and state are 16-byte aligned. Returns nonzero when
+// the state size is above 512.
 extern "C" int launch_ssd_scan(const void* xbc, long xs, const void* dt,
                                long dts, const float* dt_bias,
                                const float* rate, const float* skip,
                                float* state, const int* state_slots,
                                const int* cu, const int* positions, float* y,
-                               float* ws, float* fade, int pieces, int B,
-                               int H, int G, int N, int V, int c, int vec,
-                               hipStream_t s) {
+                               float* ws, double* logs, float* steps,
+                               float* tails, float* fade, int* table,
+                               int pieces, int B, int H, int G, int N, int V,
+                               int c, int vec, hipStream_t s) {
     if (B == 0) return 0;
     SsdArgs a{xbc, xs, dt, dts, dt_bias, rate, skip, state, state_slots, cu,
-              positions, y, ws, fade, B, H, G, N, V};
+              positions, y, ws, logs, steps, tails, fade, table, B, H, G, N,
+              V};
     if (c) return ssd_dispatch<float>(a, pieces, vec != 0, s);
     return ssd_dispatch<unsigned short>(a, pieces, vec != 0, s);
 }

@@ -1371,6 +1371,33 @@ def side_gate(g: torch.Tensor, table: torch.Tensor, offset: int,
     return (gf * e).to(g.dtype)
 
 
+def packed_attn(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor,
+                cu_seqlens: torch.Tensor, scale: float, window: int,
+                gate: Optional[torch.Tensor]) -> torch.Tensor:
+    """Causal grouped-query attention of whole prompts: q [T, H, D], k and v
+    [T, G, D], chunk b's rows cu[b] .. cu[b + 1] are positions 0, 1, ... and
+    see only each other (0 <= i - j < window when window > 0), scores
+    (q . k) * scale; head h's output times sigmoid(gate[t, h]).
+    Returns [T, H * D]."""
+    T, H, D = q.shape
+    G = k.shape[1]
+    own = torch.arange(H, device=q.device) // (H // G)
+    out = torch.zeros(T, H, v.shape[2], dtype=torch.float32, device=q.device)
+    cu = cu_seqlens.tolist()
+    for lo, hi in zip(cu, cu[1:]):
+        i = torch.arange(hi - lo, device=q.device)
+        d = i[:, None] - i[None, :]
+        dead = (d < 0) | (d >= window if window > 0 else d < 0)
+        qq = q[lo:hi].float().transpose(0, 1)
+        kk = k[lo:hi].float()[:, own].permute(1, 2, 0).contiguous()
+        s = (torch.bmm(qq, kk) * scale).masked_fill(dead, float("-inf"))
+        vv = v[lo:hi].float()[:, own].transpose(0, 1).contiguous()
+        out[lo:hi] = torch.bmm(torch.softmax(s, -1), vv).transpose(0, 1)
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())[..., None]
+    return out.reshape(T, -1).to(q.dtype)
+
+
 SSD_CHUNK = 64
 
 

@@ -180,6 +180,30 @@ def test_head_sizes_of_the_matrix_core_paths(tmp_path, dtype, kv, window,
         assert_logits(got, want, dtype)
 
 
+@pytest.mark.parametrize("window", [1, 64, 90])
+def test_whole_prompts_with_projected_keys(tmp_path, window):
+    """bf16, a latent row wider than its keys and values: whole prompts
+    project keys and values, portions and decode rows score latent rows; all
+    equal the oracle, alone and as several whole prompts in one step"""
+    cfg = O.make_config(width=64, vocab=90, lat_heads=3, lat_dim=64,
+                        lat_vdim=64, kv_rank=96, lat_window=window,
+                        lat_scale=0.125)
+    W = O.random_weights(cfg, seed=27)
+    eng = make_engine(tmp_path, cfg, W, device="cuda", dtype=torch.bfloat16,
+                      kv_blocks=60)
+    assert eng.weights.layers[1].mix[""].w_ukv is not None
+    reqs = {r: random_tokens(n, cfg["vocab"], 30 + n)
+            for r, n in (("a", 210), ("b", 5), ("c", 130))}
+    want = {r: oracle_logits(cfg, W, t) for r, t in reqs.items()}
+    for sched in ([[("a", 210), ("b", 5), ("c", 130)]],
+                  [[("a", 100), ("c", 64)], [("a", 110), ("b", 5), ("c", 66)]],
+                  [[("a", 200), ("b", 5), ("c", 129)]] +
+                  [[("a", 1)]] * 10 + [[("c", 1)]]):
+        got = replay(eng, reqs, sched)
+        for r in reqs:
+            assert_logits(got[r], want[r], torch.bfloat16, r)
+
+
 def _edge_check(tmp_path, case, dtype, sched, window, far, stays):
     cfg, W, toks = case
     T = len(toks)
@@ -218,11 +242,13 @@ def test_window_and_kept_edges_show(tmp_path, dtype, window, keep, far, dim,
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("window,far,rank", [(64, 3, 64), (17, 15, 64),
-                                             (100, 0, 8), (33, 31, 5)])
+@pytest.mark.parametrize("window,far,rank,dim", [
+    (64, 3, 64, 4), (17, 15, 64, 4), (100, 0, 8, 4), (33, 31, 5, 4),
+    (65, 2, 80, 64), (70, 63, 72, 64)])
 @pytest.mark.parametrize("sched", ["whole", "decode", "portions"])
-def test_latent_window_edge_shows(tmp_path, dtype, window, far, rank, sched):
-    case = planted_latent(window, far, far + window + 20, rank=rank)
+def test_latent_window_edge_shows(tmp_path, dtype, window, far, rank, dim,
+                                  sched):
+    case = planted_latent(window, far, far + window + 20, rank=rank, dim=dim)
     _edge_check(tmp_path, case, dtype, sched, window, far, False)
 
 

@@ -309,6 +309,55 @@ def test_latent_attention_without_rotated_part(dtype, H, C, window):
             torch.testing.assert_close(a, b, **tol(dtype))
 
 
+@pytest.mark.parametrize("H,G,D", [(4, 4, 64), (2, 1, 128), (6, 3, 64)])
+@pytest.mark.parametrize("window", [0, 1, 63, 64, 65, 200])
+def test_packed_attention(H, G, D, window):
+    """whole prompts on packed keys: windows around a key tile, prompts
+    shorter than, at and past a query tile"""
+    torch.manual_seed(10)
+    lens = [70, 1, 130, 16, 64]
+    T = sum(lens)
+    cu = torch.tensor([0] + lens, device=DEV).cumsum(0).to(torch.int32)
+    wide = torch.randn(T, (H + 2 * G) * D + 16, device=DEV).bfloat16()
+    q = wide[:, : H * D].view(T, H, D)
+    k = wide[:, H * D : (H + G) * D].view(T, G, D)
+    v = wide[:, (H + G) * D : (H + 2 * G) * D].view(T, G, D)
+    for gate in (None, sliced(T, H, torch.bfloat16, 8)):
+        a = ops.packed_attn(q, k, v, cu, 0.13, window, gate, max(lens))
+        b = ref.packed_attn(q, k, v, cu, 0.13, window, gate)
+        torch.testing.assert_close(a.float(), b.float(), rtol=2e-2, atol=3e-2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rows,I,limit", [(7, 5, 1.0), (9, 64, 0.7),
+                                          (3, 2052, 7.0)])
+def test_clamped_glu_rows(dtype, rows, I, limit):
+    torch.manual_seed(11)
+    gu = (torch.randn(rows, 2 * I, device=DEV) * 3).to(dtype)
+    torch.testing.assert_close(
+        ops.clamped_glu(gu, limit, 1.702).float(),
+        ref.clamped_glu(gu, limit, 1.702).float(), **tol(dtype))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_short_conv_many_tokens(dtype):
+    """enough tokens that a workgroup walks several of them, borders of
+    sequences inside its share"""
+    torch.manual_seed(12)
+    lens = [4001, 3, 1, 200]
+    m = batch_meta(lens, [0, 7, 1, 3], 16, 300)
+    C, taps = 40, 4
+    x = sliced(m["T"], C, dtype, 8)
+    w, b = torch.randn(taps, C, device=DEV), torch.randn(C, device=DEV)
+    st1 = torch.randn(6, taps - 1, C, device=DEV).to(dtype)
+    st2 = st1.clone()
+    args = (m["state_slots"], m["cu"], m["seq"], m["pos"], True)
+    a = ops.short_conv(x, w, st1, *args, bias=b)
+    c = ref.short_conv(x, w, st2, *args, bias=b)
+    torch.testing.assert_close(a, c, **tol(torch.float32))
+    assert torch.equal(st1, st2)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("E,ff,n,k", [(5, 10, 7, 2), (8, 64, 32, 1),
                                       (1, 4, 0, 1), (12, 20, 12, 12)])
