@@ -421,136 +421,151 @@ ssd_carry_kernel(SsdArgs a) {
     else *slot = S[0];
 }
 
-// (piece, head, 64-column block); wave w owns token rows 16w .. 16w+15 of the
-// piece and needs no other wave's results. SD_MS: LDS row stride of its masked
-// C B^T tile, written in the C layout and read back as the A operand.
+// (piece, head, 64-column block of VT 16-column tiles). First wave w forms the
+// decayed C B^T of token rows 16w .. 16w+15 in LDS, in the C layout; then every
+// wave owns one column tile of RT = VT row tiles (so a state column is read by
+// one wave), reading the LDS tile back as the A operand. SD_MS: its row stride.
 constexpr int SD_MS = SD_L + 4;
-
-// what one step of 32 state rows reads: C of the wave's tokens, B of the
-// tokens up to them, the state
-template <typename T, int VT> struct SdStep {
-    Row8<T> c, b[4];
-    float s[VT][8];
-};
 
 template <typename T, int VT, bool VEC>
 __global__ void __launch_bounds__(SD_THREADS)
 ssd_outputs_kernel(SsdArgs a) {
-    __shared__ __attribute__((aligned(16))) float ms[SD_THREADS / WAVE]
-                                                    [16 * SD_MS];
+    constexpr int RT = VT;
+    static_assert(SD_THREADS / WAVE * RT == 4 * VT, "waves cover the tiles");
+    __shared__ __attribute__((aligned(16))) float ms[SD_L * SD_MS];
     const int lo = a.table[2 * blockIdx.x], n = a.table[2 * blockIdx.x + 1];
+    if (n == 0) return;
     const int lane = threadIdx.x % WAVE;
     const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
-    const int t0 = wid * 16;
-    if (t0 >= n) return;                // no workgroup barrier below
     const int h = blockIdx.y, g = h / (a.H / a.G);
-    const int v0 = blockIdx.z * SD_L;
     const int lg = lane >> 4, li = lane & 15;
     const int N = a.N, V = a.V;
     const long hp = (long)blockIdx.x * a.H + h;
     const T* X = (const T*)a.xbc + (long)h * V;
     const T* Bp = (const T*)a.xbc + (long)a.H * V + (long)g * N;
-    const T* crow = Bp + (long)a.G * N + (long)(lo + min(t0 + li, n - 1)) * a.xs;
-    const T* brow[4];
+    const T* Cp = Bp + (long)a.G * N;
+    const double* As = a.logs + hp * SD_L;
+    const float* ds = a.steps + hp * SD_L;
+    // rows past the end repeat the last one and are not stored
+    const T *brow[4], *crow[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const long row = (long)(lo + min(j * 16 + li, n - 1)) * a.xs;
+        brow[j] = Bp + row;
+        crow[j] = Cp + row;
+    }
+    const int t0 = wid * 16;
+    // everything that needs no product yet is fetched ahead: the first step of
+    // C S, the wave's columns of X, its rows' log decays
+    const float* S = a.ws + hp * N * V;
+    const int vt = wid % VT, rt0 = wid / VT * RT;
+    // columns past the end repeat the last one and are not stored
+    const int c0 = blockIdx.z * SD_L + vt * 16 + li, col = min(c0, V - 1);
+    struct Step { Row8<T> c[RT]; float s[8]; };
+    auto load = [&](Step& st, int k) {
+        const int kc = k + lg * 8;
+        // rows of S past the end repeat the last one; C is zero there
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+            st.s[e] = S[(long)min(kc + e, N - 1) * V + col];
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+            st.c[i].template load<VEC>(crow[VT == 4 ? i : rt0 + i], kc, N);
+    };
+    Step cur, nxt;
+    load(cur, 0);
+    T xr[4][4];
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-        brow[j] = Bp + (long)(lo + min(j * 16 + li, n - 1)) * a.xs;
-    const float* S = a.ws + hp * N * V;
-    // columns past the end repeat the last one and are not stored
-    int col[VT];
 #pragma unroll
-    for (int v = 0; v < VT; ++v) col[v] = min(v0 + v * 16 + li, V - 1);
-
-    auto load = [&](SdStep<T, VT>& st, int k) {
-        const int kc = k + lg * 8;
-        st.c.template load<VEC>(crow, kc, N);
+        for (int e = 0; e < 4; ++e)
+            xr[j][e] = X[(long)(lo + min(j * 16 + lg * 4 + e, n - 1)) * a.xs +
+                         col];
+    if (t0 < n) {
+        const T* own = Cp + (long)(lo + min(t0 + li, n - 1)) * a.xs;
+        f32x4 cb[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j)     // later keys than any row: unused
-            if (j <= wid) st.b[j].template load<VEC>(brow[j], kc, N);
+        for (int j = 0; j < 4; ++j) cb[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        double At[4];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            // rows past the end repeat the last one; C is zero there
-            const float* srow = S + (long)min(kc + e, N - 1) * V;
+        for (int r = 0; r < 4; ++r) At[r] = As[t0 + lg * 4 + r];
+        struct Keys { Row8<T> c, b[4]; };
+        auto keys = [&](Keys& st, int k) {
+            st.c.template load<VEC>(own, k + lg * 8, N);
 #pragma unroll
-            for (int v = 0; v < VT; ++v) st.s[v][e] = srow[col[v]];
+            for (int j = 0; j < 4; ++j)     // tokens after every row: unused
+                if (j <= wid)
+                    st.b[j].template load<VEC>(brow[j], k + lg * 8, N);
+        };
+        Keys kc, kn;
+        keys(kc, 0);
+        for (int k = 0; k < N; k += 32) {
+            if (k + 32 < N) keys(kn, k + 32);
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                if (j <= wid) cb[j] = mma32(kc.c, kc.b[j], cb[j]);
+            kc = kn;
         }
-    };
-    f32x4 acc[VT], cb[4];
 #pragma unroll
-    for (int v = 0; v < VT; ++v) acc[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < 4; ++j) {
+            if (j > wid) continue;
+            const int s = j * 16 + li;
+            const double Asv = As[s];
+            const float d = ds[s];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) cb[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    SdStep<T, VT> cur, nxt;
-    load(cur, 0);
+            for (int r = 0; r < 4; ++r) {
+                const int t = t0 + lg * 4 + r;
+                ms[t * SD_MS + s] =
+                    s <= t ? cb[j][r] * expf((float)(At[r] - Asv)) * d : 0.f;
+            }
+        }
+    }
+    f32x4 acc[RT];
+#pragma unroll
+    for (int i = 0; i < RT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int k = 0; k < N; k += 32) {
         if (k + 32 < N) load(nxt, k + 32);
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-            if (j <= wid) cb[j] = mma32(cur.c, cur.b[j], cb[j]);
-#pragma unroll
         for (int e = 0; e < 8; ++e)
 #pragma unroll
-            for (int v = 0; v < VT; ++v)
-                acc[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    cur.c.get(e), cur.s[v][e], acc[v], 0, 0, 0);
+            for (int i = 0; i < RT; ++i)
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    cur.c[i].get(e), cur.s[e], acc[i], 0, 0, 0);
         cur = nxt;
     }
-    float* m = ms[wid];
-    const double* As = a.logs + hp * SD_L;
-    const float* ds = a.steps + hp * SD_L;
-    double At[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        At[r] = As[t0 + lg * 4 + r];
-        const float f = expf((float)At[r]);
+    for (int i = 0; i < RT; ++i)
 #pragma unroll
-        for (int v = 0; v < VT; ++v) acc[v][r] *= f;
-    }
+        for (int r = 0; r < 4; ++r)
+            acc[i][r] *= expf((float)As[(rt0 + i) * 16 + lg * 4 + r]);
+    __syncthreads();
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        if (j > wid) continue;
-        const int s = j * 16 + li;
-        const double Asv = As[s];
-        const float d = ds[s];
+        if (j * 16 >= n || j >= rt0 + RT) continue;
+#pragma unroll
+        for (int i = 0; i < RT; ++i) {
+            if (rt0 + i < j || (rt0 + i) * 16 >= n) continue;
+            const f32x4 mv = *reinterpret_cast<const f32x4*>(
+                ms + ((rt0 + i) * 16 + li) * SD_MS + j * 16 + lg * 4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    mv[e], ldf(&xr[j][e]), acc[i], 0, 0, 0);
+        }
+    }
+    if (c0 >= V) return;
+    const float skip = a.skip[h];
+    float* y = a.y + (long)lo * a.H * V + (long)h * V + col;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        // row tile j, whose X rows are the C layout's rows
+        if (j < rt0 || j >= rt0 + RT) continue;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int t = t0 + lg * 4 + r;
-            m[(lg * 4 + r) * SD_MS + s] =
-                s <= t ? cb[j][r] * expf((float)(At[r] - Asv)) * d : 0.f;
-        }
-    }
-    WAVE_LDS_SYNC();
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        if (j > wid) continue;
-        const f32x4 mv = *reinterpret_cast<const f32x4*>(
-            m + li * SD_MS + j * 16 + lg * 4);
-        float x[4][VT];
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const long row =
-                (long)(lo + min(j * 16 + lg * 4 + e, n - 1)) * a.xs;
-#pragma unroll
-            for (int v = 0; v < VT; ++v) x[e][v] = ldf(X + row + col[v]);
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e)
-#pragma unroll
-            for (int v = 0; v < VT; ++v)
-                acc[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    mv[e], x[e][v], acc[v], 0, 0, 0);
-    }
-    const float skip = a.skip[h];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-        const int t = t0 + lg * 4 + r;
-        if (t >= n) continue;
-#pragma unroll
-        for (int v = 0; v < VT; ++v) {
-            const float x = ldf(X + (long)(lo + t) * a.xs + col[v]);
-            if (v0 + v * 16 + li < V)
-                a.y[(long)(lo + t) * a.H * V + (long)h * V + col[v]] =
-                    acc[v][r] + skip * x;
+            const int t = j * 16 + lg * 4 + r;
+            if (t < n)
+                y[(long)t * a.H * V] =
+                    acc[VT == 4 ? j : j - rt0][r] + skip * ldf(&xr[j][r]);
         }
     }
 }
